@@ -143,19 +143,25 @@ struct Kernels::Fn {
   int (*cast_from_f32)(P, CP, int64_t, hipStream_t);
   int (*stream_norm_add_rounded)(P, CP, CP, CP, int, int, int, float, float, float, P, hipStream_t);
   int (*stream_norm_add_f32_rounded)(P, CP, CP, CP, int, int, int, float, float, float, P, hipStream_t);
-  int (*moe_route_scored)(P, P, P, CP, CP, CP, int, int, int, int, int, float, int, hipStream_t);
+  int (*moe_route_scored)(P, P, P, CP, CP, CP, int, int, int, int, int, float, int, int, int, float, hipStream_t);
   int (*moe_glu_weighed)(P, CP, int64_t, int, float, float, float, CP, CP, hipStream_t);
   int (*norm_columns)(P, int64_t, CP, int64_t, int, int, CP, int, float, int, hipStream_t);
   int (*gemm_heads)(P, int64_t, int64_t, CP, int64_t, int64_t, CP, int, int, int, int, hipStream_t);
-  int (*latent_post)(CP, int64_t, CP, int64_t, int64_t, int, P, P, P, CP, int, float, CP, int, CP, CP, int, int, int, int, int, int, hipStream_t);
+  int (*latent_post)(CP, int64_t, CP, int64_t, int64_t, int, P, P, P, CP, int, float, CP, float, int, CP, CP, int, int, int, int, int, int, hipStream_t);
   int (*qkv_post_norm_angles_paired)(CP, int64_t, P, P, P, CP, CP, int, int, float, CP, float, int, int, CP, CP, int, int, int, int, int, hipStream_t);
   int (*linear_rule)(P, CP, int64_t, int, int, int, CP, P, int64_t, CP, CP, CP, int, int, int, int, float, hipStream_t);
   int (*side_gate)(P, int64_t, CP, int64_t, CP, int64_t, CP, int, int, int, hipStream_t);
   int (*gated_row_norm)(P, int64_t, CP, CP, int64_t, CP, int, int, int, float, int, hipStream_t);
   int (*silu_columns)(P, int64_t, int64_t, int, int, hipStream_t);
+  int (*hyper_in_place)(int, int);
+  int (*hyper_step)(CP, int, P, CP, int, CP, CP, P, P, CP, int, float, int, int, int, hipStream_t);
+  int (*hyper_close)(P, CP, int, CP, int, CP, CP, int, int, int, hipStream_t);
+  int (*embed_normed)(P, CP, CP, CP, int, int, int, int, float, hipStream_t);
+  int (*attention_wide)(P, CP, CP, CP, CP, int, CP, CP, CP, int, int, int, int, int, int, int, float, CP, int, hipStream_t);
+  int (*attention_wide_limit)();
 };
 
-static constexpr int KERNEL_ABI = 18;
+static constexpr int KERNEL_ABI = 19;
 
 Kernels::Kernels(const std::string& lib_dir, const std::string& name) : name_(name), fn_(new Fn) {
   if (name == "bf16") dtype_ = DType::BF16;
@@ -198,6 +204,8 @@ Kernels::Kernels(const std::string& lib_dir, const std::string& name) : name_(na
   VK(norm_columns, "vk_norm_columns"); VK(gemm_heads, "vk_gemm_heads"); VK(latent_post, "vk_latent_post");
   VK(qkv_post_norm_angles_paired, "vk_qkv_post_norm_angles_paired"); VK(linear_rule, "vk_linear_rule"); VK(side_gate, "vk_side_gate");
   VK(gated_row_norm, "vk_gated_row_norm"); VK(silu_columns, "vk_silu_columns");
+  VK(hyper_in_place, "vk_hyper_in_place"); VK(hyper_step, "vk_hyper_step"); VK(hyper_close, "vk_hyper_close"); VK(embed_normed, "vk_embed_normed");
+  VK(attention_wide, "vk_attention_wide"); VK(attention_wide_limit, "vk_attention_wide_limit");
 #undef VK
   segment_keys_ = fn_->attn_segment_keys();
   item_rows_ = fn_->attn_item_rows();
@@ -584,6 +592,12 @@ void Kernels::paged_attention_capped(Tensor& out, const Tensor& q, const Tensor&
   if (sinks) sf = norm_weight(*sinks, "attention sinks", nq);
   void* sp = nullptr;
   const int64_t n_items = items.dim(0);
+  if (d > 256) {
+    if (keep != 0 || block != 0 || softcap != 0.f) throw EngineError("attention: rows of more than 256 entries are built without kept keys, blocks and caps");
+    call(fn_->attention_wide(out.data, q.data, k_cache.data, v_cache.data, block_table.data, (int)W, cu_q.data, k_len.data, items.data, (int)n_items,
+                             mode == 1 ? 1 : item_rows_, (int)nq, (int)nkv, (int)d, (int)P, window, scale, sinks ? sinks->data : nullptr, sf, stream));
+    return;
+  }
   if (mode == 1) {
     if (nseg < (max_k_len + segment_keys_ - 1) / segment_keys_)
       throw EngineError("attention: " + std::to_string(nseg) + " segments do not cover " + std::to_string(max_k_len) + " keys");
@@ -881,7 +895,7 @@ Kernels::MoePlan Kernels::moe_route(const Tensor& h, const Tensor& router, int t
 }
 
 Kernels::MoePlan Kernels::moe_route_scored(const Tensor& h, const Tensor& router, int top, float weight_eps, int tile_rows, const Tensor* bias,
-                                           int score_kind) {
+                                           int score_kind, int groups, int keep, float scale) {
   expect(h, "router input", dtype_);
   expect(router, "router weight", dtype_);
   if (h.shape.size() != 2 || router.shape.size() != 2 || router.dim(1) != h.dim(1) || top < 1 || top > router.dim(0))
@@ -901,10 +915,10 @@ Kernels::MoePlan Kernels::moe_route_scored(const Tensor& h, const Tensor& router
   p.tile_expert = empty({tiles}, DType::I32);
   p.expert_start = empty({E + 1}, DType::I32);
   Tensor logits = empty({T, E}, DType::F32);
-  if (score_kind != 0) {
+  if (score_kind != 0 || groups != 1 || scale != 1.f) {
     const int bf = bias ? norm_weight(*bias, "router bias", E) : 0;
     call(fn_->moe_route_scored(p.idx.data, p.wts.data, logits.data, h.data, router.data, bias ? bias->data : nullptr, bf, (int)T, (int)h.dim(1), (int)E,
-                               top, weight_eps, score_kind, stream));
+                               top, weight_eps, score_kind, groups, keep, scale, stream));
   } else if (bias) {
     const int bf = norm_weight(*bias, "router bias", E);
     call(fn_->moe_route_bias(p.idx.data, p.wts.data, logits.data, h.data, router.data, bias->data, bf, (int)T, (int)h.dim(1), (int)E, top, weight_eps,
@@ -1010,7 +1024,7 @@ void Kernels::gemm_heads(Tensor& out, int64_t out_stride, const Tensor& x, int64
 }
 
 void Kernels::latent_post(const Tensor& proj, int64_t kv_col, const Tensor& q, int64_t q_stride, int64_t q_first, Tensor& q_abs, const Tensor* k_cache,
-                          const Tensor* v_cache, int page_size, const Tensor* norm_w, float eps, const Tensor& inv_freq, bool neighbours,
+                          const Tensor* v_cache, int page_size, const Tensor* norm_w, float eps, const Tensor& inv_freq, float mag, bool neighbours,
                           const Tensor& positions, const Tensor* slots, int r, int dr) {
   expect(q, "queries", dtype_);
   expect(q_abs, "queries as the cache meets them", dtype_);
@@ -1036,9 +1050,59 @@ void Kernels::latent_post(const Tensor& proj, int64_t kv_col, const Tensor& q, i
   }
   call(fn_->latent_post(store ? static_cast<const char*>(proj.data) + (size_t)kv_col * dtype_bytes(dtype_) : nullptr, store ? proj.dim(1) : 0, q.data,
                         q.dim(1), q_stride, (int)q_first, q_abs.data, store ? k_cache->data : nullptr, store ? v_cache->data : nullptr,
-                        store ? norm_w->data : nullptr, wf, eps, inv_freq.data, neighbours ? 1 : 0, positions.data, store ? slots->data : nullptr, (int)T,
+                        store ? norm_w->data : nullptr, wf, eps, inv_freq.data, mag, neighbours ? 1 : 0, positions.data, store ? slots->data : nullptr, (int)T,
                         (int)H, r, dr, (int)D, page_size, stream));
 }
+
+// ------------------------------------------------------------------ a residual of several streams
+Tensor Kernels::embed_normed(const Tensor& table, const Tensor& ids, const Tensor& w, float eps) {
+  expect(table, "embedding table", dtype_);
+  if (table.shape.size() != 2) throw EngineError("embedding table is " + table.describe());
+  const int64_t V = table.dim(0), H = table.dim(1), T = ids.numel();
+  expect(ids, "ids", DType::I32, {T});
+  const int wf = norm_weight(w, "embedding norm weight", H);
+  Tensor out = empty({T, H}, DType::F32);
+  call(fn_->embed_normed(out.data, table.data, ids.data, w.data, wf, (int)T, (int)H, (int)V, eps, stream));
+  return out;
+}
+
+// What the two launches on streams share: the streams' shape, the output that is written back and its coefficients.
+static bool hyper_one_row(const Tensor& streams, int S, const Tensor* y, const Tensor* back, DType elem) {
+  const size_t rank = streams.shape.size();
+  if (streams.dtype != DType::F32 || S < 1 || (rank != 2 && (rank != 3 || streams.dim(1) != S)))
+    throw EngineError("hyper-connections: " + std::to_string(S) + " streams are " + streams.describe());
+  if (y && (y->shape != std::vector<int64_t>{streams.dim(0), streams.dim(-1)} || (y->dtype != DType::F32 && y->dtype != elem)))
+    throw EngineError("hyper-connections: an output " + y->describe() + " for streams " + streams.describe());
+  if (y && (!back || back->dtype != DType::F32 || back->numel() != (int64_t)S * (S + 2))) throw EngineError("hyper-connections: an output without its coefficients");
+  return rank == 2;
+}
+
+Tensor Kernels::hyper_step(Tensor& streams, const Tensor* y, const Tensor* back, const Tensor& take, int S, const Tensor* w, float eps) {
+  const bool one = hyper_one_row(streams, S, y, back, dtype_);
+  const int64_t T = streams.dim(0), W = streams.dim(-1);
+  expect(take, "hyper-connections' coefficients", DType::F32, {(int64_t)S * (S + 2)});
+  const int wf = w ? norm_weight(*w, "norm weight", W) : 0;
+  Tensor next = streams;
+  if (y && (one || !fn_->hyper_in_place((int)W, S))) next = empty({T, (int64_t)S, W}, DType::F32);
+  Tensor out = w ? empty({T, W}) : empty({T, W}, DType::F32);
+  call(fn_->hyper_step(static_cast<const float*>(streams.data), one ? 1 : 0, y ? next.data : nullptr, y ? y->data : nullptr,
+                       y && y->dtype == DType::F32 ? 1 : 0, y ? back->data : nullptr, take.data, w ? out.data : nullptr, w ? nullptr : out.data,
+                       w ? w->data : nullptr, wf, eps, (int)T, (int)W, S, stream));
+  streams = next;
+  return out;
+}
+
+Tensor Kernels::hyper_close(const Tensor& streams, const Tensor* y, const Tensor* back, int S, const Tensor& rows) {
+  const bool one = hyper_one_row(streams, S, y, back, dtype_);
+  const int64_t R = rows.numel(), W = streams.dim(-1);
+  expect(rows, "rows", DType::I32, {R});
+  Tensor out = empty({R, W}, DType::F32);
+  call(fn_->hyper_close(out.data, streams.data, one ? 1 : 0, y ? y->data : nullptr, y && y->dtype == DType::F32 ? 1 : 0, y ? back->data : nullptr,
+                        rows.data, (int)R, (int)W, S, stream));
+  return out;
+}
+
+int Kernels::attention_limit() const { return fn_->attention_wide_limit(); }
 
 Tensor Kernels::qkv_post_norm_angles_paired(const Tensor& qkv, int nq, int nkv, int d, const Tensor* k_cache, const Tensor* v_cache, int page_size,
                                             const Tensor* q_w, const Tensor* k_w, int norm_d, float eps, const Tensor& inv_freq, float mag,

@@ -232,7 +232,10 @@ class Kernels {
   Tensor gemm_grouped(const Tensor& act, const Tensor& w, const Tensor& block_weights);
   bool gemm_grouped_takes(int64_t K) const;
   // moe_route with a choice of score: 0 as moe_route; 1: a chosen expert's weight is the logistic function of its logit.
-  MoePlan moe_route_scored(const Tensor& h, const Tensor& router, int top, float weight_eps, int tile_rows, const Tensor* bias, int score_kind);
+  // 2: the softmax over all experts as it is.  groups, keep: only experts of the `keep` best of that many equal groups can be
+  // chosen; scale: on every weight.
+  MoePlan moe_route_scored(const Tensor& h, const Tensor& router, int top, float weight_eps, int tile_rows, const Tensor* bias, int score_kind,
+                           int groups = 1, int keep = 1, float scale = 1.f);
   // moe_glu for experts that read their input times the pair's weight: every row's gate and up values are multiplied by
   // its pair's weight before the clamps; moe_sum_unweighed then adds a token's rows as they are.
   Tensor moe_glu_weighed(const Tensor& gate_up, float limit, float slope, float shift, const MoePlan& plan);
@@ -243,9 +246,9 @@ class Kernels {
   // out[:, h * out_stride : + N] = x[:, x_col + h * x_stride : + K] W[h]^T for every head; w [H, N, K]; out [T, out_width] elements.
   void gemm_heads(Tensor& out, int64_t out_stride, const Tensor& x, int64_t x_col, int64_t x_stride, const Tensor& w);
   // The latent's norm, the rotation of the key part and of the heads' rotated query parts, and the cache store, in one
-  // launch.  q_abs [T, H, D]: its columns [r, D) of every head are written.  kv_col < 0: queries only.
+  // launch.  q_abs [T, H, D]: its columns [r, D) of every head are written.  kv_col < 0: queries only.  mag: on every cosine and sine.
   void latent_post(const Tensor& proj, int64_t kv_col, const Tensor& q, int64_t q_stride, int64_t q_first, Tensor& q_abs, const Tensor* k_cache,
-                   const Tensor* v_cache, int page_size, const Tensor* norm_w, float eps, const Tensor& inv_freq, bool neighbours,
+                   const Tensor* v_cache, int page_size, const Tensor* norm_w, float eps, const Tensor& inv_freq, float mag, bool neighbours,
                    const Tensor& positions, const Tensor* slots, int r, int dr);
   // qkv_post_norm_angles with a choice of pairs: neighbours true turns elements 2c and 2c + 1; the norms may be absent.
   Tensor qkv_post_norm_angles_paired(const Tensor& qkv, int nq, int nkv, int d, const Tensor* k_cache, const Tensor* v_cache, int page_size,
@@ -263,6 +266,18 @@ class Kernels {
   // ---- a token's slice of a second embedding table, gated (stream.hip)
   // gelu(gate[:, 0:n]) * table[ids, first : first + n] as elements [T, gate.dim(1)], zero beyond n.
   Tensor side_gate(const Tensor& gate, const Tensor& table, const Tensor& ids, int64_t first, int64_t n);
+  // ---- a residual of several streams in 32-bit (hyper.hip)
+  // table[ids] / sqrt(mean(.^2) + eps) * w as floats [T, width].
+  Tensor embed_normed(const Tensor& table, const Tensor& ids, const Tensor& w, float eps);
+  // Writes a sublayer's output y [T, W] (elements or floats; null: there is none) back into the streams and reads the next
+  // sublayer's input.  streams: [T, S, W] floats, or [T, W] where all streams are still one row; it holds the new streams
+  // afterwards.  back, take: floats [a: S | b: S | M: S * S] of the sublayer that gave y and of the next one.  Returns
+  // norm(u) * w as elements, or (w null) u as floats.
+  Tensor hyper_step(Tensor& streams, const Tensor* y, const Tensor* back, const Tensor& take, int S, const Tensor* w, float eps);
+  // The sum of the streams of the rows that are asked for, after the last output: floats [rows, W].
+  Tensor hyper_close(const Tensor& streams, const Tensor* y, const Tensor* back, int S, const Tensor& rows);
+  // The widest cached row that attention takes; rows of more than 256 entries go through vector arithmetic.
+  int attention_limit() const;
   void relu_square(Tensor& x);                 // x <- max(x, 0)^2
   int segment_keys() const { return segment_keys_; }
   int item_rows() const { return item_rows_; }

@@ -5,6 +5,7 @@
 #include <cstring>
 #include <set>
 #include <sstream>
+#include <tuple>
 
 namespace vosti {
 
@@ -339,14 +340,11 @@ Tensor DecoderModel::forward(const Tensor& ids, StepContext& ctx, std::vector<Ca
     residual = hr.second;
   }
   if (want_rows.numel() == 0) return kernels_.empty({0, spec_.vocab_size});
-  hidden = kernels_.gather_rows(hidden, want_rows);
+  if (spec_.schedule.empty()) hidden = kernels_.gather_rows(hidden, want_rows);
+  else std::tie(hidden, residual) = layers_[spec_.schedule.back().layer]->rows_for_the_end(hidden, residual, ctx, want_rows);
   Tensor normed;
-  if (residual.data == nullptr) {
-    normed = final_norm_->forward(hidden);            // a model without layers
-  } else {
-    Tensor r = kernels_.gather_rows(residual, want_rows);
-    normed = final_norm_->forward_add(hidden, r);
-  }
+  if (residual.data == nullptr) normed = final_norm_->forward(hidden);            // nothing is left to add
+  else normed = final_norm_->forward_add(hidden, residual);
   return head_->forward(normed);
 }
 

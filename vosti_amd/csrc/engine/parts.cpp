@@ -6,6 +6,7 @@
 
 #include <algorithm>
 #include <cmath>
+#include <cstring>
 #include <mutex>
 
 namespace vosti {
@@ -90,6 +91,11 @@ std::pair<Tensor, Tensor> PositionEncoding::apply(const Tensor& q, const Tensor&
     return kernels.qkv_post(x.view({T, n * d}), (int)n, 0, (int)d, nullptr, nullptr, 0, nullptr, nullptr, 0.f, cos, sin, &positions, nullptr);
   };
   return {rotate(q), k.data ? rotate(k) : Tensor()};
+}
+
+std::pair<Tensor, Tensor> Block::rows_for_the_end(const Tensor& hidden, const Tensor& residual, StepContext& ctx, const Tensor& rows) {
+  (void)ctx;
+  return {kernels.gather_rows(hidden, rows), residual.data ? kernels.gather_rows(residual, rows) : Tensor()};
 }
 
 void Norm::forward_scaled_add(const Tensor& y, const Tensor& base, Tensor& out, float mult, Tensor* rounded) {
@@ -192,6 +198,23 @@ Tensor pad_column_blocks(const Tensor& w, int64_t n, int64_t size, int64_t size_
   return out;
 }
 
+// A weight's elements as floats on the host.
+std::vector<float> host_floats(const Tensor& w) {
+  std::vector<float> out((size_t)w.numel());
+  if (w.dtype == DType::F32) {
+    hip_check(hipMemcpy(out.data(), w.data, w.bytes(), hipMemcpyDeviceToHost), "reading a weight back");
+    return out;
+  }
+  if (w.dtype != DType::BF16) throw EngineError("a weight of " + w.describe() + " holds no floats");
+  std::vector<uint16_t> raw(out.size());
+  hip_check(hipMemcpy(raw.data(), w.data, w.bytes(), hipMemcpyDeviceToHost), "reading a weight back");
+  for (size_t i = 0; i < raw.size(); ++i) {
+    const uint32_t b = (uint32_t)raw[i] << 16;
+    std::memcpy(&out[i], &b, 4);
+  }
+  return out;
+}
+
 int64_t round_up(int64_t n, int64_t to) { return (n + to - 1) / to * to; }
 
 // h[t] = E[ids[t]], a row copy without scale (src/exec/dense_swiglu_model.rs:271-273).
@@ -246,6 +269,27 @@ class ScaledEmbedding : public Embedding {
   int64_t vocab_, hidden_;
   float scale_;
   Tensor weight_;
+};
+
+// h[t] = E[ids[t]] / sqrt(mean(.^2) + eps) * w, as the residual stream in 32-bit whatever the element type.
+class NormedEmbedding : public Embedding {
+ public:
+  NormedEmbedding(const PartSpec& s, Kernels& k)
+      : Embedding(k), vocab_(s.integer("vocab_size")), hidden_(s.integer("hidden_size")), eps_((float)s.number("eps")) {}
+  std::vector<ParamDecl> params() const override {
+    ParamDecl w{"norm.weight", {hidden_}, true, true, 0.9, 1.1};
+    return {{"weight", {vocab_, hidden_}}, w};
+  }
+  void load(std::map<std::string, Tensor>& t) override {
+    weight_ = need(t, "weight");
+    norm_ = need(t, "norm.weight");
+  }
+  Tensor forward(const Tensor& ids) override { return kernels.embed_normed(weight_, ids, norm_, eps_); }
+
+ private:
+  int64_t vocab_, hidden_;
+  float eps_;
+  Tensor weight_, norm_;
 };
 
 // y = (x * rsqrt(mean(x^2) + eps)) * w in 32-bit (kernels/triton_kernels/rmsnorm.py:63-93); with a residual
@@ -1151,7 +1195,10 @@ class PairMean : public Mixer {
 // shared_size (> 0: one more expert of that inner size and the same form, with shared_limit, that every token uses
 // with weight 1; its output is added to the sum), score (1: the weights are the logistic function of the chosen logits, not
 // divided by anything), weigh_input (1: the output is the sum of expert(weight * h); since W (w h) = w (W h), the weight
-// multiplies the gate and up outputs before their clamps, and the sum adds the experts' outputs as they are).
+// multiplies the gate and up outputs before their clamps, and the sum adds the experts' outputs as they are; score 2: the
+// weights are the softmax scores over all experts as they are), groups and keep_groups (the experts form that many equal runs of
+// neighbours, a group's score is its largest, and only experts of the best keep_groups can be chosen), weight_scale (on every
+// weight).  limit absent: nothing is clamped.
 class RoutedExperts : public FeedForward {
  public:
   RoutedExperts(const PartSpec& s, Kernels& k)
@@ -1159,8 +1206,14 @@ class RoutedExperts : public FeedForward {
         top_((int)s.integer("top")), weight_eps_((float)s.number("weight_eps", 0.0)), bias_(s.integer("router_bias", 0) != 0),
         gated_(s.integer("gated", 0) != 0), limit_((float)s.number("limit", 0.0)), slope_((float)s.number("glu_slope", 1.0)),
         shift_((float)s.number("up_shift", 0.0)), shared_(s.integer("shared_size", 0)), shared_limit_((float)s.number("shared_limit", 0.0)),
-        score_((int)s.integer("score", 0)), weigh_input_(s.integer("weigh_input", 0) != 0) {
-    if (score_ < 0 || score_ > 1) throw ConfigError("experts: 'score' is 0 (softmax) or 1 (the logistic function of a chosen logit)");
+        score_((int)s.integer("score", 0)), weigh_input_(s.integer("weigh_input", 0) != 0), groups_((int)s.integer("groups", 1)),
+        keep_((int)s.integer("keep_groups", 1)), weight_scale_((float)s.number("weight_scale", 1.0)) {
+    if (score_ < 0 || score_ > 2)
+      throw ConfigError("experts: 'score' is 0 (softmax, divided by the chosen sum), 1 (the logistic function of a chosen logit) or 2 (softmax as it is)");
+    if (groups_ < 1 || experts_ % groups_ || keep_ < 1 || keep_ > groups_ || top_ > keep_ * (experts_ / groups_))
+      throw ConfigError("experts: " + std::to_string(experts_) + " in " + std::to_string(groups_) + " groups of which " + std::to_string(keep_) +
+                        " are kept cannot give " + std::to_string(top_));
+    if (gated_ && !s.numbers.count("limit")) limit_ = INFINITY;
     if (weigh_input_ && (!gated_ || shared_ > 0)) throw ConfigError("experts whose weights scale their inputs are built in the gated form, without a shared expert");
     if (experts_ < 1 || top_ < 1 || top_ > experts_) throw ConfigError("a mixture of " + std::to_string(experts_) + " experts cannot choose " + std::to_string(top_));
     if (gated_ && !(limit_ > 0.f)) throw ConfigError("gated experts need a positive 'limit'");
@@ -1217,13 +1270,13 @@ class RoutedExperts : public FeedForward {
     // the rows are sorted by expert into blocks of 128 and go through the engine's tile product, every block with its
     // expert's matrix.  Both are launched from numbers on the GPU alone and give the same bits.
     if (pairs < (int64_t)kRowsAnExpertForTiles * experts_ || !k.gemm_grouped_takes(hidden_) || !k.gemm_grouped_takes(w_down_.dim(2))) {
-      const Kernels::MoePlan plan = k.moe_route_scored(x, router_, top_, weight_eps_, 16, bias, score_);
+      const Kernels::MoePlan plan = k.moe_route_scored(x, router_, top_, weight_eps_, 16, bias, score_, groups_, keep_, weight_scale_);
       if (weigh_input_)
         return k.moe_sum_unweighed(k.moe_down(k.moe_glu_weighed(k.moe_up_plain(x, w_up_, plan), limit_, slope_, shift_, plan), w_down_, plan), plan);
       const Tensor act = gated_ ? k.moe_glu(k.moe_up_plain(x, w_up_, plan), limit_, slope_, shift_) : k.moe_up(x, w_up_, plan);
       return k.moe_sum(k.moe_down(act, w_down_, plan), plan, extra);
     }
-    const Kernels::MoePlan plan = k.moe_route_scored(x, router_, top_, weight_eps_, 128, bias, score_);
+    const Kernels::MoePlan plan = k.moe_route_scored(x, router_, top_, weight_eps_, 128, bias, score_, groups_, keep_, weight_scale_);
     Tensor act = k.gemm_grouped(k.gather_rows(x, plan.row_token), w_up_, plan.tile_expert);
     if (weigh_input_) return k.moe_sum_unweighed(k.gemm_grouped(k.moe_glu_weighed(act, limit_, slope_, shift_, plan), w_down_, plan.tile_expert), plan);
     if (gated_) act = k.moe_glu(act, limit_, slope_, shift_);
@@ -1240,8 +1293,10 @@ class RoutedExperts : public FeedForward {
   float limit_, slope_, shift_;
   int64_t shared_;
   float shared_limit_;
-  int score_;              // 0: softmax scores; 1: a chosen expert's weight is the logistic function of its logit
+  int score_;              // 0: softmax scores over their chosen sum; 1: the logistic function of a chosen logit; 2: softmax scores as they are
   bool weigh_input_;       // a weight scales what its expert reads (the gate and up outputs before their clamps), not what it gives
+  int groups_, keep_;      // experts of the best keep_ of groups_ equal groups can be chosen
+  float weight_scale_;
   Tensor router_, router_bias_, w_up_, w_down_, w_shared_in_, w_shared_down_;
 };
 
@@ -1308,10 +1363,12 @@ Tensor rearranged(const Tensor& w, int64_t rows, int64_t cols, const std::functi
 
 // Attention through a latent.  For the mixer's input h, with H heads, per head d entries that are not rotated and dr that
 // are, value size dv, latent size r and query latent size rq:
-//   c_q = norm(W_dq h) (weight dq.norm), q = W_uq c_q, head by head [d | dr];  W_dkv h = [latent: r | key part: dr];
+//   c_q = norm(W_dq h) (weight dq.norm), q = W_uq c_q, head by head [d | dr] (q_rank 0: q = W_q h, no latent of its own);
+//   W_dkv h = [latent: r | key part: dr];
 //   c = norm(latent) (weight dkv.norm); the key part is rotated by the position and serves every head;
 //   head j: k_j = W_uk[j] c, v_j = W_uv[j] c; score = (q_flat . k_j + rotate(q_rot) . rotated key part) * scale;
-//   softmax over the keys so far; the heads side by side times sigmoid(W_g h); then W_o.
+//   softmax over the keys so far (window > 0: that many last keys; sink 1: exp of a learned number per head joins the
+//   denominator); the heads side by side, times sigmoid(W_g h) with output_gate 1; then W_o.
 // Only c and the rotated key part are kept: the cache has one kv head whose key row is [c | rotated part | 0] and whose
 // value row is [c | 0], D = r + dr rounded up to 16 entries.  Since q_flat . (W_uk[j] c) = (W_uk[j]^T q_flat) . c, head j's
 // query meets the cache as [W_uk[j]^T q_flat | rotate(q_rot) | 0], and its output is W_uv[j] times the weighted sum of the
@@ -1324,10 +1381,13 @@ class LatentAttention : public Mixer {
   LatentAttention(const PartSpec& s, Kernels& k)
       : Mixer(k), hidden_(s.integer("hidden_size")), H_((int)s.integer("num_heads")), d_((int)s.integer("head_dim")), dr_((int)s.integer("rotary_dim")),
         dv_((int)s.integer("value_dim")), r_((int)s.integer("kv_rank")), rq_((int)s.integer("q_rank")), scale_((float)s.number("scale")),
-        eps_((float)s.number("eps")), own_kv_(s.integer("own_kv", 1) != 0), gate_(s.integer("output_gate", 0) != 0) {
+        eps_((float)s.number("eps")), own_kv_(s.integer("own_kv", 1) != 0), gate_(s.integer("output_gate", 0) != 0),
+        window_((int)s.integer("window", 0)), sink_(s.integer("sink", 0) != 0) {
     D_ = (int)round_up((int64_t)r_ + dr_, 16);
-    if (H_ < 1 || d_ < 1 || dr_ < 2 || dr_ % 2 || dv_ < 1 || r_ < 1 || rq_ < 1) throw ConfigError("latent attention: bad sizes");
-    if (D_ > 256) throw ConfigError("latent attention: a latent of " + std::to_string(r_) + " with " + std::to_string(dr_) + " rotated entries: the attention kernels take up to 256 together");
+    if (H_ < 1 || d_ < 1 || dr_ < 2 || dr_ % 2 || dv_ < 1 || r_ < 1 || rq_ < 0 || window_ < 0) throw ConfigError("latent attention: bad sizes");
+    if (D_ > k.attention_limit())
+      throw ConfigError("latent attention: a latent of " + std::to_string(r_) + " with " + std::to_string(dr_) + " rotated entries: the attention kernels take up to " +
+                        std::to_string(k.attention_limit()) + " together");
     const PartSpec* p = s.part("position");
     if (!p) throw ConfigError("latent attention needs the part 'position'");
     position_ = build_part<PositionEncoding>("position", *p, k);
@@ -1339,10 +1399,19 @@ class LatentAttention : public Mixer {
   }
   std::vector<ParamDecl> params() const override {
     ParamDecl qn{"q_down_norm.weight", {(int64_t)rq_}, true, true, 0.9, 1.1}, kn{"kv_down_norm.weight", {(int64_t)r_}, true, true, 0.9, 1.1};
-    ParamDecl uq{"q_up.weight", {(int64_t)H_ * (d_ + dr_), (int64_t)rq_}}, uk{"k_up.weight", {(int64_t)H_ * d_, (int64_t)r_}},
+    ParamDecl uq{rq_ ? "q_up.weight" : "q_proj.weight", {(int64_t)H_ * (d_ + dr_), rq_ ? (int64_t)rq_ : hidden_}}, uk{"k_up.weight", {(int64_t)H_ * d_, (int64_t)r_}},
         uv{"v_up.weight", {(int64_t)H_ * dv_, (int64_t)r_}};
-    uq.p0 = uk.p0 = uv.p0 = 0.06;
-    std::vector<ParamDecl> p = {{"q_down.weight", {(int64_t)rq_, hidden_}}, qn, uq, uk, uv, {"o_proj.weight", {hidden_, (int64_t)H_ * dv_}}};
+    uk.p0 = uv.p0 = 0.06;
+    if (rq_) uq.p0 = 0.06;
+    std::vector<ParamDecl> p = {uq, uk, uv, {"o_proj.weight", {hidden_, (int64_t)H_ * dv_}}};
+    if (rq_) {
+      p.push_back({"q_down.weight", {(int64_t)rq_, hidden_}});
+      p.push_back(qn);
+    }
+    if (sink_) {
+      ParamDecl sinks{"sinks", {(int64_t)H_}, true, true, -1.0, 1.0};
+      p.push_back(sinks);
+    }
     if (own_kv_) {
       p.push_back({"kv_down.weight", {(int64_t)r_ + dr_, hidden_}});
       p.push_back(kn);
@@ -1353,24 +1422,32 @@ class LatentAttention : public Mixer {
   std::vector<std::pair<std::string, Part*>> children() override { return {{"position", position_.get()}}; }
   void load(std::map<std::string, Tensor>& t) override {
     if (!position_->angle_frequencies()) throw ConfigError("latent attention is built for rotations by computed angles");
-    // One launch projects the query's latent, the latent with its key part (where the layer has them) and the gate.
-    std::vector<Tensor> rows = {pad_matrix(need(t, "q_down.weight"), rqp_, hidden_)};
+    const int64_t d = d_, dr = dr_, dp = dp_, qs = qs_, r = r_, dv = dv_, D = D_;
+    // A head's query rows as [d | zeros to dp | dr | zeros to qs], the columns padded to the padded latent.
+    auto query_rows = [&](const Tensor& w, int64_t cols, int64_t cols_to) {
+      if (dp == d && qs == d + dr && cols == cols_to) return w;
+      return rearranged(w, (int64_t)H_ * qs, cols_to, [=](int64_t i, int64_t j) -> std::pair<int64_t, int64_t> {
+        const int64_t h = i / qs, e = i % qs;
+        if (j >= cols) return {-1, 0};
+        if (e < d) return {h * (d + dr) + e, j};
+        if (e >= dp && e < dp + dr) return {h * (d + dr) + d + (e - dp), j};
+        return {-1, 0};
+      });
+    };
+    // One launch projects the queries or their latent, the latent with its key part (where the layer has them) and the gate.
+    std::vector<Tensor> rows = {rq_ ? pad_matrix(need(t, "q_down.weight"), rqp_, hidden_) : query_rows(need(t, "q_proj.weight"), hidden_, hidden_)};
     if (own_kv_) rows.push_back(pad_matrix(need(t, "kv_down.weight"), kvp_, hidden_));
     if (gate_) rows.push_back(pad_row_blocks(need(t, "gate_proj.weight"), H_, dv_, dvp_));
     w_in_ = rows.size() > 1 ? stack_rows(rows) : rows[0];
-    kv_col_ = own_kv_ ? rqp_ : -1;
-    gate_col_ = rqp_ + (own_kv_ ? kvp_ : 0);
-    q_norm_ = need(t, "q_down_norm.weight");
+    const int64_t q_rows = rows[0].dim(0);
+    kv_col_ = own_kv_ ? q_rows : -1;
+    gate_col_ = q_rows + (own_kv_ ? kvp_ : 0);
+    if (rq_) {
+      q_norm_ = need(t, "q_down_norm.weight");
+      w_uq_ = query_rows(need(t, "q_up.weight"), rq_, rqp_);
+    }
+    if (sink_) sinks_ = need(t, "sinks");
     if (own_kv_) kv_norm_ = need(t, "kv_down_norm.weight");
-    const int64_t d = d_, dr = dr_, dp = dp_, qs = qs_, r = r_, dv = dv_, D = D_;
-    // A head's query rows as [d | zeros to dp | dr | zeros to qs], the columns padded to the padded latent.
-    w_uq_ = rearranged(need(t, "q_up.weight"), (int64_t)H_ * qs, rqp_, [=](int64_t i, int64_t j) -> std::pair<int64_t, int64_t> {
-      const int64_t h = i / qs, e = i % qs;
-      if (j >= rq_) return {-1, 0};
-      if (e < d) return {h * (d + dr) + e, j};
-      if (e >= dp && e < dp + dr) return {h * (d + dr) + d + (e - dp), j};
-      return {-1, 0};
-    });
     // Head h's W_uk transposed: [r, dp], so that a product a head takes q_flat to the latent's side.
     w_absorb_ = rearranged(need(t, "k_up.weight"), (int64_t)H_ * r, dp, [=](int64_t i, int64_t j) -> std::pair<int64_t, int64_t> {
                   if (j >= d) return {-1, 0};
@@ -1390,6 +1467,7 @@ class LatentAttention : public Mixer {
     n.kind = CacheNeed::Pages;
     n.num_kv_heads = 1;
     n.head_dim = D_;
+    n.window = window_;
     return n;
   }
   const char* step_inputs_key() const override { return "attention.items"; }
@@ -1409,22 +1487,23 @@ class LatentAttention : public Mixer {
     const int64_t T = x.dim(0);
     GroupTables& tables = ctx.groups.at(cache.group);
     const Tensor proj = k.gemm(x, w_in_);
-    const Tensor q = k.gemm(k.norm_columns(proj, 0, rq_, q_norm_, eps_, rqp_), w_uq_);
+    const Tensor q = rq_ ? k.gemm(k.norm_columns(proj, 0, rq_, q_norm_, eps_, rqp_), w_uq_) : proj;
     Tensor q_abs = k.empty({T, (int64_t)H_, (int64_t)D_});
     Tensor q_abs_rows = q_abs.view({T, (int64_t)H_ * D_});
     k.gemm_heads(q_abs_rows, D_, q, 0, qs_, w_absorb_);
     k.latent_post(proj, kv_col_, q, qs_, dp_, q_abs, &cache.k, &cache.v, cache.page_size, own_kv_ ? &kv_norm_ : nullptr, eps_,
-                  *position_->angle_frequencies(), position_->pairs_neighbours(), ctx.positions, &tables.slots, r_, dr_);
+                  *position_->angle_frequencies(), position_->magnitude(), position_->pairs_neighbours(), ctx.positions, &tables.slots, r_, dr_);
+    const Tensor* sinks = sink_ ? &sinks_ : nullptr;
     Tensor out = k.empty(q_abs.shape);
     AttentionItems& m = attention_items(k, *ctx.host);
     const Tensor& prefill_items = ctx.inputs.at("attention.prefill_items");
     const Tensor& decode_items = ctx.inputs.at("attention.decode_items");
     if (prefill_items.dim(0))
-      k.paged_attention_capped(out, q_abs, cache.k, cache.v, tables.block_table, ctx.cu_q, ctx.k_len, prefill_items, 0, scale_, 0, 0, 0.f, nullptr,
+      k.paged_attention_capped(out, q_abs, cache.k, cache.v, tables.block_table, ctx.cu_q, ctx.k_len, prefill_items, 0, scale_, window_, 0, 0.f, sinks,
                                ctx.host->k_len_bound, 0, nullptr, 0);
     if (decode_items.dim(0)) {
       const Tensor scratch = ctx.workspace(k.attn_scratch_floats((int)decode_items.dim(0), H_, D_, m.nseg));
-      k.paged_attention_capped(out, q_abs, cache.k, cache.v, tables.block_table, ctx.cu_q, ctx.k_len, decode_items, 1, scale_, 0, 0, 0.f, nullptr,
+      k.paged_attention_capped(out, q_abs, cache.k, cache.v, tables.block_table, ctx.cu_q, ctx.k_len, decode_items, 1, scale_, window_, 0, 0.f, sinks,
                                m.decode_bound, m.nseg, &scratch, 0);
     }
     Tensor heads = k.empty({T, (int64_t)H_ * dvp_});
@@ -1438,9 +1517,11 @@ class LatentAttention : public Mixer {
   int H_, d_, dr_, dv_, r_, rq_, D_ = 0;       // D_: the head size of the cache and the attention kernels
   float scale_, eps_;
   bool own_kv_, gate_;
+  int window_;
+  bool sink_;
   int64_t dp_ = 0, qs_ = 0, rqp_ = 0, kvp_ = 0, dvp_ = 0, kv_col_ = -1, gate_col_ = 0;
   std::unique_ptr<PositionEncoding> position_;
-  Tensor w_in_, w_uq_, w_absorb_, w_expand_, w_o_, q_norm_, kv_norm_;
+  Tensor w_in_, w_uq_, w_absorb_, w_expand_, w_o_, q_norm_, kv_norm_, sinks_;
 };
 
 // Linear attention with one fixed decay a head.  For the mixer's input h:
@@ -1606,6 +1687,100 @@ class PostNormBlock : public Block {
   bool has_ffn_ = true;
 };
 
+// A residual of `streams` copies in 32-bit that start equal (hyper-connections).  Around each sublayer (the mixer; then the
+// feed-forward, if the layer has one), with its coefficients in (S), out (S) and mix (S x S, [from, to]):
+//   u = sum over s of in[s] x_s;  y = sublayer(norm(u));  x_t <- sum over s of mix[s, t] x_s + out[t] y.
+// Writing an output back and reading the next input are one launch over the streams (Kernels::hyper_step), also from one
+// layer to the next: a layer leaves its last output and that sublayer's coefficients in ctx.carry, the next layer's first
+// launch writes them back, and after the last layer rows_for_the_end() does, while it adds the streams of the rows that are
+// asked for.
+class HyperStreamsBlock : public Block {
+ public:
+  HyperStreamsBlock(Kernels& k, std::unique_ptr<Mixer> mixer, std::unique_ptr<FeedForward> ffn, std::map<std::string, std::unique_ptr<Norm>> norms,
+                    const std::map<std::string, double>& numbers)
+      : Block(k), mixer_(std::move(mixer)), ffn_(std::move(ffn)), norms_(std::move(norms)) {
+    auto number = [&](const char* name) {
+      auto it = numbers.find(name);
+      if (it == numbers.end()) throw ConfigError(std::string("a hyper_streams block needs the number '") + name + "'");
+      return (int64_t)it->second;
+    };
+    hidden_ = number("hidden_size");
+    S_ = (int)number("streams");
+    if (S_ < 1 || S_ > 64) throw ConfigError("a hyper_streams block of " + std::to_string(S_) + " streams: 1 to 64 are built");
+    has_ffn_ = dynamic_cast<NoFeedForward*>(ffn_.get()) == nullptr;
+    if (!norms_.count("mixer_in")) throw ConfigError("a hyper_streams block needs the norm 'mixer_in'");
+    if (has_ffn_ && !norms_.count("ffn_in")) throw ConfigError("a hyper_streams block with a feed-forward needs the norm 'ffn_in'");
+  }
+  std::vector<ParamDecl> params() const override {
+    std::vector<ParamDecl> p;
+    for (const char* sub : {"hyper_mixer.", "hyper_ffn."}) {
+      if (sub == std::string("hyper_ffn.") && !has_ffn_) continue;
+      ParamDecl in{std::string(sub) + "in", {(int64_t)S_}, true, true, 0.5, 1.0}, out{std::string(sub) + "out", {(int64_t)S_}, true, true, 0.7, 1.3},
+          mix{std::string(sub) + "mix", {(int64_t)S_, (int64_t)S_}, true, true, 0.5 / S_, 1.5 / S_};
+      p.insert(p.end(), {in, out, mix});
+    }
+    return p;
+  }
+  void load(std::map<std::string, Tensor>& t) override {
+    mixer_coef_ = coefficients(t, "hyper_mixer.");
+    if (has_ffn_) ffn_coef_ = coefficients(t, "hyper_ffn.");
+  }
+  std::vector<std::pair<std::string, Part*>> children() override {
+    std::vector<std::pair<std::string, Part*>> c = {{"mixer", mixer_.get()}, {"feed_forward", ffn_.get()}};
+    for (auto& n : norms_) c.emplace_back("norms." + n.first, n.second.get());
+    return c;
+  }
+  Mixer& mixer() override { return *mixer_; }
+  std::pair<Tensor, Tensor> forward(const Tensor& hidden, Tensor residual, StepContext& ctx, CacheEntry& cache) override {
+    Tensor streams = hidden;
+    const Tensor pending = left(ctx, hidden), back = pending.data ? ctx.carry["hyper.back"] : Tensor();
+    Tensor y = mixer_->forward(read(streams, pending.data ? &pending : nullptr, &back, mixer_coef_, *norms_["mixer_in"]), ctx, cache);
+    if (has_ffn_) y = ffn_->forward(read(streams, &y, &mixer_coef_, ffn_coef_, *norms_["ffn_in"]), ctx);
+    ctx.carry["hyper.output"] = y;
+    ctx.carry["hyper.back"] = has_ffn_ ? ffn_coef_ : mixer_coef_;
+    ctx.carry["hyper.of"] = streams;
+    return {streams, residual};
+  }
+  std::pair<Tensor, Tensor> rows_for_the_end(const Tensor& hidden, const Tensor&, StepContext& ctx, const Tensor& rows) override {
+    const Tensor pending = left(ctx, hidden), back = pending.data ? ctx.carry["hyper.back"] : Tensor();
+    return {kernels.hyper_close(hidden, pending.data ? &pending : nullptr, &back, S_, rows), Tensor()};
+  }
+
+ private:
+  // The output that the layer before left unwritten; none before a step's first layer.
+  Tensor left(StepContext& ctx, const Tensor& streams) const {
+    if (streams.dtype != DType::F32 || streams.dim(0) != ctx.num_tokens || streams.dim(-1) != hidden_)
+      throw EngineError("a hyper_streams block takes the 32-bit residual streams, not " + streams.describe());
+    auto it = ctx.carry.find("hyper.output");
+    if (it == ctx.carry.end()) return Tensor();
+    if (ctx.carry["hyper.of"].data != streams.data) throw EngineError("a hyper_streams block was handed other streams than the layer before left");
+    return it->second;
+  }
+  Tensor read(Tensor& streams, const Tensor* y, const Tensor* back, const Tensor& take, Norm& norm) {
+    if (const Tensor* w = norm.row_scale_weight()) return kernels.hyper_step(streams, y, back, take, S_, w, norm.eps());
+    return norm.forward(kernels.hyper_step(streams, y, back, take, S_, nullptr, 0.f));
+  }
+  // A sublayer's coefficients as one row of floats: in, out, mix.
+  Tensor coefficients(std::map<std::string, Tensor>& t, const std::string& prefix) const {
+    std::vector<float> all;
+    for (const char* n : {"in", "out", "mix"}) {
+      const std::vector<float> v = host_floats(need(t, prefix + n));
+      all.insert(all.end(), v.begin(), v.end());
+    }
+    Tensor out = zero_weight({(int64_t)all.size()}, DType::F32);
+    hip_check(hipMemcpy(out.data, all.data(), all.size() * sizeof(float), hipMemcpyHostToDevice), "hyper-connections' coefficients");
+    return out;
+  }
+
+  std::unique_ptr<Mixer> mixer_;
+  std::unique_ptr<FeedForward> ffn_;
+  std::map<std::string, std::unique_ptr<Norm>> norms_;
+  int64_t hidden_ = 0;
+  int S_ = 1;
+  bool has_ffn_ = true;
+  Tensor mixer_coef_, ffn_coef_;
+};
+
 template <class T>
 PartFactory factory() {
   return [](const PartSpec& s, Kernels& k) { return std::unique_ptr<Part>(new T(s, k)); };
@@ -1646,6 +1821,11 @@ void register_standard_parts() {
     register_block("post_norm", [](Kernels& k, std::unique_ptr<Mixer> m, std::unique_ptr<FeedForward> f,
                                    std::map<std::string, std::unique_ptr<Norm>> n, const std::map<std::string, double>& numbers) {
       return std::unique_ptr<Block>(new PostNormBlock(k, std::move(m), std::move(f), std::move(n), numbers));
+    });
+    register_part("embedding", "token_embedding_normed", factory<NormedEmbedding>());
+    register_block("hyper_streams", [](Kernels& k, std::unique_ptr<Mixer> m, std::unique_ptr<FeedForward> f,
+                                       std::map<std::string, std::unique_ptr<Norm>> n, const std::map<std::string, double>& numbers) {
+      return std::unique_ptr<Block>(new HyperStreamsBlock(k, std::move(m), std::move(f), std::move(n), numbers));
     });
     register_part("norm", "rmsnorm", factory<RMSNorm>());
     register_part("position", "rotary", factory<Rotary>());

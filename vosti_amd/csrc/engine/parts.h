@@ -159,6 +159,9 @@ class Block : public Part {
   virtual Mixer& mixer() = 0;
   // (hidden, residual) -> (hidden, residual); `residual` has no memory before the first layer.
   virtual std::pair<Tensor, Tensor> forward(const Tensor& hidden, Tensor residual, StepContext& ctx, CacheEntry& cache) = 0;
+  // The rows of (hidden, residual) that the model's end reads, asked of the last layer that ran.  An arrangement that keeps
+  // the stream in another form between layers brings it into the form of the final norm here.
+  virtual std::pair<Tensor, Tensor> rows_for_the_end(const Tensor& hidden, const Tensor& residual, StepContext& ctx, const Tensor& rows);
 };
 
 using PartFactory = std::function<std::unique_ptr<Part>(const PartSpec&, Kernels&)>;

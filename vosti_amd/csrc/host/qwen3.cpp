@@ -9,6 +9,7 @@
 
 #include "qwen3.h"
 #include "pabavik.h"
+#include "kelisun.h"
 #include "pasovik.h"
 #include "povatar.h"
 #include "tezinex.h"
@@ -196,6 +197,7 @@ void register_builtin_architectures() {
   register_architecture("Povatar", "povatar", povatar_model_spec);
   register_architecture("Pabavik", "pabavik", pabavik_model_spec);
   register_architecture("Pasovik", "pasovik", pasovik_model_spec);
+  register_architecture("Kelisun", "kelisun", kelisun_model_spec);
 }
 
 }  // namespace vosti

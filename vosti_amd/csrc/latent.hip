@@ -105,17 +105,18 @@ struct LatentPostArgs {
   const int32_t* positions;
   const int32_t* slots;   // page * P + offset, or -1
   int H, r, dr, D, P, neighbours;
-  float eps;
+  float eps, mag;         // mag: the factor on every cosine and sine
 };
 
 // Element j of a part of dr entries after its rotation: pair c is the entries 2c and 2c + 1 (neighbours) or c and c + dr/2.
-__device__ __forceinline__ float rotated_entry(const elem_t* part, int j, int dr, int neighbours, float posf, const float* __restrict__ inv_freq) {
+__device__ __forceinline__ float rotated_entry(const elem_t* part, int j, int dr, int neighbours, float posf, const float* __restrict__ inv_freq,
+                                               float mag) {
   const int half = dr / 2;
   const int pair = neighbours ? j >> 1 : (j < half ? j : j - half);
   const bool second = neighbours ? (j & 1) != 0 : j >= half;
   const int other = neighbours ? (j ^ 1) : (second ? j - half : j + half);
   const float angle = posf * inv_freq[pair];
-  const float cs = cosf(angle), sn = sinf(angle);
+  const float cs = cosf(angle) * mag, sn = sinf(angle) * mag;
   const float mine = to_f32(part[j]), theirs = to_f32(part[other]);
   return second ? mine * cs + theirs * sn : mine * cs - theirs * sn;
 }
@@ -130,7 +131,7 @@ __global__ __launch_bounds__(256) void latent_post_kernel(LatentPostArgs a) {
   for (int i = tid; i < a.H * tail; i += 256) {
     const int h = i / tail, j = i - h * tail;
     const elem_t* part = a.q + (int64_t)t * a.ldq + (int64_t)h * a.qs + a.q_first;
-    const float v = j < a.dr ? rotated_entry(part, j, a.dr, a.neighbours, posf, a.inv_freq) : 0.f;
+    const float v = j < a.dr ? rotated_entry(part, j, a.dr, a.neighbours, posf, a.inv_freq, a.mag) : 0.f;
     a.q_out[((int64_t)t * a.H + h) * a.D + a.r + j] = from_f32<elem_t>(v);
   }
   if (a.kv == nullptr) return;
@@ -152,7 +153,7 @@ __global__ __launch_bounds__(256) void latent_post_kernel(LatentPostArgs a) {
     if (c < a.r) {
       kval = vval = (to_f32(row[c]) * rr) * load_weight(a.w, a.w_is_f32, c);
     } else {
-      kval = c < a.r + a.dr ? rotated_entry(row + a.r, c - a.r, a.dr, a.neighbours, posf, a.inv_freq) : 0.f;
+      kval = c < a.r + a.dr ? rotated_entry(row + a.r, c - a.r, a.dr, a.neighbours, posf, a.inv_freq, a.mag) : 0.f;
       vval = 0.f;
     }
     krow[c] = from_f32<elem_t>(kval);
@@ -186,7 +187,7 @@ int vk_gemm_heads(elem_t* out, int64_t ldo, int64_t os, const elem_t* x, int64_t
 
 // kv null: the layer reads another's cache, and only the queries are written.
 int vk_latent_post(const elem_t* kv, int64_t ldkv, const elem_t* q, int64_t ldq, int64_t qs, int q_first, elem_t* q_out, elem_t* kc, elem_t* vc,
-                   const void* w, int w_is_f32, float eps, const float* inv_freq, int neighbours, const int32_t* positions, const int32_t* slots, int T,
+                   const void* w, int w_is_f32, float eps, const float* inv_freq, float mag, int neighbours, const int32_t* positions, const int32_t* slots, int T,
                    int H, int r, int dr, int D, int P, hipStream_t st) {
   VK_REQUIRE(T >= 0 && H > 0 && r > 0 && dr > 0 && dr % 2 == 0 && D >= r + dr, "latent attention: bad sizes H=%d r=%d dr=%d D=%d", H, r, dr, D);
   VK_REQUIRE(q != nullptr && q_out != nullptr && inv_freq != nullptr && positions != nullptr && qs >= q_first + dr && ldq >= (int64_t)(H - 1) * qs + q_first + dr,
@@ -198,6 +199,7 @@ int vk_latent_post(const elem_t* kv, int64_t ldkv, const elem_t* q, int64_t ldq,
   LatentPostArgs a;
   a.kv = kv; a.ldkv = ldkv; a.q = q; a.ldq = ldq; a.qs = qs; a.q_first = q_first; a.q_out = q_out; a.kc = kc; a.vc = vc; a.w = w; a.w_is_f32 = w_is_f32;
   a.inv_freq = inv_freq; a.positions = positions; a.slots = slots; a.H = H; a.r = r; a.dr = dr; a.D = D; a.P = P; a.neighbours = neighbours; a.eps = eps;
+  a.mag = mag;
   latent_post_kernel<<<T, 256, 0, st>>>(a);
   return vk_check_launch("latent attention");
 }

@@ -61,12 +61,38 @@ __global__ __launch_bounds__(256) void moe_logits_kernel(float* __restrict__ z, 
   }
 }
 
+// LDS traffic between the lanes of a wave: what was written before is read after.
+__device__ __forceinline__ void wave_lds_fence() {
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+}
+
+// The place of the largest of v[0 .. n) over a wave (the lower index wins a tie; values above -2).
+__device__ __forceinline__ int wave_argmax(const float* v, int n, int lane, float& best) {
+  best = -2.f;
+  int at = 0x7fffffff;
+  for (int i = lane; i < n; i += 64) {
+    const float x = v[i];
+    if (x > best) { best = x; at = i; }
+  }
+#pragma unroll
+  for (int off = 32; off >= 1; off >>= 1) {
+    const float ov = __shfl_xor(best, off, VK_WAVE);
+    const int oe = __shfl_xor(at, off, VK_WAVE);
+    if (ov > best || (ov == best && oe < at)) { best = ov; at = oe; }
+  }
+  return min(at, n - 1);        // scores that are no numbers must not become an address
+}
+
 // The choice: idx [T, top] int32, wts [T, top] floats from the logits.  One wave per token, four tokens a workgroup.
 // score 0: the softmax over all experts, the chosen scores divided by their sum plus weight_eps; score 1: the logistic
-// function of every logit, the chosen scores as they are (the order of the scores is the order of the logits either way).
+// function of every logit, the chosen scores as they are (the order of the scores is the order of the logits either way);
+// score 2: the softmax over all experts, the chosen scores as they are.  Every weight is multiplied by `scale` at the end.
+// groups > 1 with keep < groups: the experts form that many equal runs of neighbours; a group's score is its largest, and
+// only experts of the `keep` best groups can be chosen.
 __global__ __launch_bounds__(256) void moe_choose_kernel(int32_t* __restrict__ idx, float* __restrict__ wts, const float* __restrict__ logits,
-                                                         int T, int E, int top, float weight_eps, int score_kind) {
-  extern __shared__ float scores[];      // [4][E]
+                                                         int T, int E, int top, float weight_eps, int score_kind, int groups, int keep, float scale) {
+  extern __shared__ float scores[];      // [4][E], then [4][groups]
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int t = blockIdx.x * 4 + wave;
   if (t >= T) return;
@@ -84,36 +110,47 @@ __global__ __launch_bounds__(256) void moe_choose_kernel(int32_t* __restrict__ i
     sum = sum + p;
   }
   sum = score_kind == 1 ? 1.f : wave_sum_xor(sum);
+  if (keep < groups) {
+    // A kept group's score is marked with -1; the experts of the others are then marked as if they had been chosen.
+    float* gs = scores + 4 * E + wave * groups;
+    const int size = E / groups;
+    wave_lds_fence();
+    for (int g = lane; g < groups; g += 64) {
+      float m = -1.f;
+      for (int j = 0; j < size; ++j) m = fmaxf(m, z[g * size + j]);
+      gs[g] = fmaxf(m, 0.f);
+    }
+    wave_lds_fence();
+    for (int k = 0; k < keep; ++k) {
+      float best;
+      const int g = wave_argmax(gs, groups, lane, best);
+      if (lane == 0) gs[g] = -1.f;
+      wave_lds_fence();
+    }
+    for (int e = lane; e < E; e += 64)
+      if (gs[e / size] >= 0.f) z[e] = -1.f;
+    wave_lds_fence();
+  }
   // The largest score `top` times; a chosen one is marked with -1 (scores are positive or zero).
   float chosen_sum = 0.f;
   float my_w = 0.f;
   int my_e = 0;
   for (int k = 0; k < top; ++k) {
-    float best = -2.f;
-    int best_e = 0x7fffffff;
-    for (int e = lane; e < E; e += 64) {
-      const float v = z[e];
-      if (v > best) { best = v; best_e = e; }
-    }
-#pragma unroll
-    for (int off = 32; off >= 1; off >>= 1) {
-      const float ov = __shfl_xor(best, off, VK_WAVE);
-      const int oe = __shfl_xor(best_e, off, VK_WAVE);
-      if (ov > best || (ov == best && oe < best_e)) { best = ov; best_e = oe; }
-    }
+    float best;
+    const int best_e = wave_argmax(z, E, lane, best);
     const float score = best / sum;
     chosen_sum = chosen_sum + score;
     if (lane == k % 64 && k < 64) { my_w = score; my_e = best_e; }
     if (k >= 64 && lane == 0) { idx[(int64_t)t * top + k] = best_e; wts[(int64_t)t * top + k] = score; }
     if (lane == 0) z[best_e] = -1.f;
-    __builtin_amdgcn_wave_barrier();
+    wave_lds_fence();
   }
-  const float denom = score_kind == 1 ? 1.f : chosen_sum + weight_eps;
+  const float denom = score_kind == 0 ? chosen_sum + weight_eps : 1.f;
   if (lane < top) {
     idx[(int64_t)t * top + lane] = my_e;
-    wts[(int64_t)t * top + lane] = my_w / denom;
+    wts[(int64_t)t * top + lane] = (my_w / denom) * scale;
   }
-  for (int k = 64 + lane; k < top; k += 64) wts[(int64_t)t * top + k] = wts[(int64_t)t * top + k] / denom;
+  for (int k = 64 + lane; k < top; k += 64) wts[(int64_t)t * top + k] = (wts[(int64_t)t * top + k] / denom) * scale;
 }
 
 // The plan, by one workgroup.  counts the pairs of every expert, gives expert e the rows [start_e, start_e + tile_rows *
@@ -320,14 +357,18 @@ int vk_moe_max_tiles(int T, int top, int E, int tile_rows) {
 
 // logits: scratch [T, E] floats.  bias [E] (elements, or floats with bias_is_f32) or null.
 static int route_launch(int32_t* idx, float* wts, float* logits, const elem_t* h, const elem_t* router, const void* bias, int bias_is_f32, int T, int W,
-                        int E, int top, float weight_eps, hipStream_t st, int score_kind = 0) {
+                        int E, int top, float weight_eps, hipStream_t st, int score_kind = 0, int groups = 1, int keep = 1, float scale = 1.f) {
   VK_REQUIRE(T >= 0 && W > 0 && W % VK_VEC == 0 && E > 0 && top > 0 && top <= E && E <= 4096,
              "router: bad sizes T=%d W=%d E=%d top=%d (the width in whole 16-byte vectors, at most 4096 experts)", T, W, E, top);
   VK_REQUIRE(((uintptr_t)h % 16) == 0 && ((uintptr_t)router % 16) == 0, "router: operands must be 16-byte aligned");
+  VK_REQUIRE(groups > 0 && E % groups == 0 && keep > 0 && keep <= groups && top <= keep * (E / groups),
+             "router: %d experts in %d groups of which %d are kept cannot give %d choices", E, groups, keep, top);
   if (T == 0) return 0;
   moe_logits_kernel<<<dim3((T + MOE_ROUTE_TOKENS - 1) / MOE_ROUTE_TOKENS, E), 256, 0, st>>>(logits, h, router, T, W, E, bias, bias_is_f32);
   if (vk_check_launch("router (logits)")) return 1;
-  moe_choose_kernel<<<(T + 3) / 4, 256, (size_t)4 * E * sizeof(float), st>>>(idx, wts, logits, T, E, top, weight_eps, score_kind);
+  const size_t lds = (size_t)4 * (E + (keep < groups ? groups : 0)) * sizeof(float);
+  VK_REQUIRE(lds <= 65536, "router: %d experts in %d groups are too many", E, groups);
+  moe_choose_kernel<<<(T + 3) / 4, 256, lds, st>>>(idx, wts, logits, T, E, top, weight_eps, score_kind, groups, keep, scale);
   return vk_check_launch("router (choice)");
 }
 
@@ -345,11 +386,13 @@ int vk_moe_route_bias(int32_t* idx, float* wts, float* logits, const elem_t* h, 
 }
 
 // The same with a choice of score: 0 is vk_moe_route (vk_moe_route_bias with a bias), 1 gives every chosen expert the
-// logistic function of its logit as its weight, not divided by anything.  bias may be null.
+// logistic function of its logit as its weight, not divided by anything, 2 the softmax over all experts as it is.  bias may be
+// null.  groups, keep: only experts of the `keep` best of that many equal groups can be chosen (1, 1: all); scale: on every
+// weight.
 int vk_moe_route_scored(int32_t* idx, float* wts, float* logits, const elem_t* h, const elem_t* router, const void* bias, int bias_is_f32, int T, int W,
-                        int E, int top, float weight_eps, int score_kind, hipStream_t st) {
-  VK_REQUIRE(score_kind == 0 || score_kind == 1, "router: score kind %d", score_kind);
-  return route_launch(idx, wts, logits, h, router, bias, bias_is_f32, T, W, E, top, weight_eps, st, score_kind);
+                        int E, int top, float weight_eps, int score_kind, int groups, int keep, float scale, hipStream_t st) {
+  VK_REQUIRE(score_kind >= 0 && score_kind <= 2, "router: score kind %d", score_kind);
+  return route_launch(idx, wts, logits, h, router, bias, bias_is_f32, T, W, E, top, weight_eps, st, score_kind, groups, keep, scale);
 }
 
 int vk_moe_plan(const int32_t* idx, int32_t* row_pair, int32_t* row_token, int32_t* pair_row, int32_t* tile_expert, int32_t* expert_start, int T,
