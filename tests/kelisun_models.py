@@ -43,17 +43,15 @@ def config(layers, width=64, vocab=97, streams=2, eps=1e-5):
 # tile has rows, one head, windows shorter than a page, equal to one and longer, stretched and plain rotations, layers
 # without a feed-forward, one expert of one, all experts chosen, one group of several, three of five; three layers that
 # share weights, one of them with a layer that comes later.
-_M = [
-    layer(latent(3, 12, 6, 20, kv_rank=20, window=10, base=500.0, scaling=(3.0, 40, 8.0, 0.5)), moe(3, 3, 40, scale=1.5)),
-    layer(latent(18, 8, 4, 8, kv_rank=16, window=33, scaling=(8.0, 64, 16.0, 1.0))),
-]
+_LATER = layer(latent(18, 8, 4, 8, kv_rank=16, window=33, scaling=(8.0, 64, 16.0, 1.0)))
+_M = [layer(latent(3, 12, 6, 20, kv_rank=20, window=10, base=500.0, scaling=(3.0, 40, 8.0, 0.5)), moe(3, 3, 40, scale=1.5)),
+      dict(_LATER, weights_of=5)]
 _M += [again(_M, 0), layer(latent(2, 16, 16, 40, kv_rank=48, window=64, base=77.0, scale=0.3), moe(1, 1, 16, scale=0.7))]
-_M += [None, again(_M, 1),
+_M += [again(_M, 3), _LATER,
        # The two routers that choose stand last: where two experts all but tie, the 16-bit engine may choose the other one,
        # and a token that went to another expert in an early layer would change the keys that later tokens read.
        layer(latent(1, 24, 10, 24, kv_rank=13, window=16, base=900.0), moe(10, 3, 24, groups=(5, 3), scale=2.5)),
        layer(latent(4, 10, 8, 12, kv_rank=30, window=21, scaling=(2.0, 100, 4.0, 1.0)), moe(8, 2, 12, groups=(2, 1)))]
-_M[4] = again(_M, 7)
 MIXED = config(_M, width=64, vocab=97, streams=3)
 # A cached row that fills the widest shared tiles of one size, one that fills the widest of all, and one between; a width
 # whose vectors do not fill a wave; two streams.
@@ -83,7 +81,7 @@ def random_weights(cfg, seed):
         m = spec["mixer"]
         H, d, dr, dv, r = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
         w[p + "norm1"] = uniform(W, lo=0.5, hi=1.5)
-        w[p + "mix.q"] = normal(H * (d + dr), W, std=1.5 * W ** -0.5)
+        w[p + "mix.q"] = normal(H * (d + dr), W, std=W ** -0.5)
         w[p + "mix.dkv"] = normal(r + dr, W, std=W ** -0.5)
         w[p + "mix.dkv.norm"] = uniform(r, lo=0.5, hi=2.0)
         w[p + "mix.uk"] = normal(H * d, r, std=r ** -0.5)
@@ -103,7 +101,9 @@ def random_weights(cfg, seed):
                 w[p + f"mlp.e{e}.down"] = normal(W, F, std=F ** -0.5)
         for s in subs:
             w[p + s + "in"] = uniform(S, lo=0.3, hi=1.2)
-            w[p + s + "out"] = uniform(S, lo=0.4, hi=1.4)
+            # The experts write less than the attention: an expert chosen otherwise by the 16-bit engine, where two all but
+            # tie, then moves a row less (in 32-bit every row is held to rounding anyway).
+            w[p + s + "out"] = uniform(S, lo=0.4, hi=1.4) if s == "hc1." else uniform(S, lo=0.2, hi=0.5)
             w[p + s + "mix"] = torch.eye(S) * 0.9 + uniform(S, S, lo=-0.3, hi=0.3)
     # What the file stores is what both sides compute with.
     return {n: t.to(torch.bfloat16).contiguous() for n, t in w.items()}

@@ -22,19 +22,19 @@ def test_description_of_a_configuration():
     spec = c.model_spec()
     # Five layers with weights of their own, run eight times, every run with a cache of its own.
     assert [l.block for l in spec.layers] == ["hyper_streams"] * 5
-    assert [l.feed_forward.kind for l in spec.layers] == ["routed_experts", "none", "routed_experts", "routed_experts", "routed_experts"]
-    assert [(e.layer, e.cache_from) for e in spec.schedule] == [(0, None), (1, None), (0, None), (2, None), (4, None), (1, None), (3, None), (4, None)]
+    assert [l.feed_forward.kind for l in spec.layers] == ["routed_experts", "routed_experts", "none", "routed_experts", "routed_experts"]
+    assert [(e.layer, e.cache_from) for e in spec.schedule] == [(0, None), (2, None), (0, None), (1, None), (1, None), (2, None), (3, None), (4, None)]
     assert spec.embedding.kind == "token_embedding_normed" and spec.embedding.params["eps"] == 1e-5
     assert spec.final_norm.params == {"size": 64, "eps": 1e-5} and "softcap" not in spec.head.params
     f = spec.layers[3].feed_forward.params
     assert (f["experts"], f["top"], f["intermediate_size"], f["gated"], f["score"], f["groups"], f["keep_groups"], f["weight_scale"]) == (10, 3, 24, 1, 2, 5, 3, 2.5)
     assert not {"limit", "router_bias", "shared_size", "weigh_input", "up_shift", "glu_slope"} & set(f)
     assert (spec.layers[0].feed_forward.params["groups"], spec.layers[0].feed_forward.params["keep_groups"]) == (1, 1)
-    n = spec.layers[4].names                               # the sixth and seventh entries' neighbour: layer 7 of the file
+    n = spec.layers[4].names
     assert n["mixer.q_proj.weight"] == "l7.mix.q" and n["mixer.kv_down_norm.weight"] == "l7.mix.dkv.norm" and n["mixer.sinks"] == "l7.mix.sink"
     assert n["norms.mixer_in.weight"] == "l7.norm1" and n["norms.ffn_in.weight"] == "l7.norm2"
     assert n["hyper_mixer.in"] == "l7.hc1.in" and n["hyper_ffn.mix"] == "l7.hc2.mix" and n["feed_forward.experts.7.down_proj.weight"] == "l7.mlp.e7.down"
-    assert "norms.ffn_in.weight" not in spec.layers[1].names and "hyper_ffn.in" not in spec.layers[1].names
+    assert "norms.ffn_in.weight" not in spec.layers[2].names and "hyper_ffn.in" not in spec.layers[2].names
 
 
 def test_the_parts_in_the_library_s_own_words():
@@ -48,21 +48,22 @@ def test_the_parts_in_the_library_s_own_words():
     r = a["parts"]["position"]
     assert r["kind"] == "rotary_stretched" and "neighbours" not in r["numbers"]
     assert [r["numbers"][k] for k in ("rotary_dim", "theta", "factor", "original", "fast", "slow")] == [6, 500, 3, 40, 8, 0.5]
-    plain_rot = d["layers"][2]["mixer"]["parts"]["position"]["numbers"]
+    plain_rot = d["layers"][1]["mixer"]["parts"]["position"]["numbers"]
     assert plain_rot["theta"] == 77 and "factor" not in plain_rot
     assert d["layers"][0]["block_numbers"] == {"hidden_size": 64, "streams": 3}
-    assert d["ignored_names"] == ["l1.norm2", "l1.hc2.in", "l1.hc2.out", "l1.hc2.mix"]
+    assert d["ignored_names"] == ["l5.norm2", "l5.hc2.in", "l5.hc2.out", "l5.hc2.mix"]
     assert d["names"]["embedding.norm.weight"] == "embed.norm" and d["names"]["head.weight"] == "head"
     # A layer without a mask sees every earlier key.
     free = json.loads(json.dumps(MIXED))
-    del free["layers"][3]["mixer"]["mask"]
-    assert describe(free)["layers"][2]["mixer"]["numbers"]["window"] == 0
+    for i in (3, 4):
+        del free["layers"][i]["mixer"]["mask"]
+    assert describe(free)["layers"][1]["mixer"]["numbers"]["window"] == 0
 
 
 @pytest.mark.parametrize("change, text", [
-    (lambda c: c["layers"][1].update(type="serial"), "unknown mixer type"),
-    (lambda c: c["layers"][1].pop("type"), "type"),
-    (lambda c: c["layers"][1].pop("mixer"), "mixer"),
+    (lambda c: c["layers"][5].update(type="serial"), "unknown mixer type"),
+    (lambda c: c["layers"][5].pop("type"), "type"),
+    (lambda c: c["layers"][5].pop("mixer"), "mixer"),
     (lambda c: c["layers"][3]["mixer"].update(heads=0), "heads"),
     (lambda c: c["layers"][3]["mixer"]["rot"].update(dims=8), "rot_dim"),
     (lambda c: c["layers"][3]["mixer"].update(rot_dim=5, rot={"base": 10.0, "dims": 5}), "even"),
