@@ -6,6 +6,7 @@
     python bench.py --workload mixed14b     # Qwen3-14B shape: 32 prompts of 128 to 4,096 tokens, prefill in portions beside decoding
     python bench.py --workload prefix32b    # Qwen3-32B shape: 64 requests at context 8,192 that share a 1,024-token prefix
     python bench.py --workload aligned      # the reference's aligned phases: batch 4, cached contexts 0 to 16K, 256 new tokens / 127 decode steps
+    python bench.py --workload kelisun      # the Kelisun design (windowed attention through a latent, experts chosen by groups, four residual streams, layers that share weights) at three layer sizes beside Pasovik at equal size
     python bench.py --workload pasovik      # the Pasovik design (attention through a latent, linear attention with fixed decays, a second embedding a layer) at three layer sizes beside Pabavik at equal size
     python bench.py --workload pabavik      # the Pabavik design (gated linear attention, windowed attention with an output gate, gated experts beside a shared one) at three layer sizes beside Tezinex at equal size
     python bench.py --workload povatar      # the Povatar design (attention beside a state-space recurrence, routed experts) at three layer sizes beside Tezinex at equal size
@@ -89,9 +90,9 @@ def main() -> int:
     ap.add_argument("--no-other-shapes", action="store_true", help="skip the 14B and 32B workloads that the default record holds as points")
     ap.add_argument("--prompt-tokens", type=int, default=PROMPT_TOKENS,
                     help="context length of the decode measurement (the prefill figure is always of 2,048 tokens)")
-    ap.add_argument("--workload", default="decode8b", choices=["decode8b", "mixed14b", "prefix32b", "aligned", "tezinex", "povatar", "pabavik", "pasovik"])
-    ap.add_argument("--sizes", default=",".join(["1k", "2k", "4k"]), help="which layer sizes --workload tezinex / povatar / pabavik / pasovik measure (1k, 2k, 4k)")
-    ap.add_argument("--only-design", default="", choices=["", "tezinex", "qwen3", "povatar", "pabavik", "pasovik"], help="--workload tezinex / povatar / pabavik / pasovik: measure one of the two designs only")
+    ap.add_argument("--workload", default="decode8b", choices=["decode8b", "mixed14b", "prefix32b", "aligned", "tezinex", "povatar", "pabavik", "pasovik", "kelisun"])
+    ap.add_argument("--sizes", default=",".join(["1k", "2k", "4k"]), help="which layer sizes --workload tezinex / povatar / pabavik / pasovik / kelisun measure (1k, 2k, 4k)")
+    ap.add_argument("--only-design", default="", choices=["", "tezinex", "qwen3", "povatar", "pabavik", "pasovik", "kelisun"], help="--workload tezinex / povatar / pabavik / pasovik / kelisun: measure one of the two designs only")
     ap.add_argument("--engine", default="native", choices=["native", "python"],
                     help="which engine every figure is measured through: the native one (vosti_amd.engine.NativeEngine) or the "
                          "Python step function over the same kernels, cache manager and scheduler")
@@ -114,7 +115,7 @@ def main() -> int:
     if args.workload == "aligned":
         print(json.dumps(aligned_workload(args)), flush=True)
         return 0
-    if args.workload in ("tezinex", "povatar", "pabavik", "pasovik"):
+    if args.workload in ("tezinex", "povatar", "pabavik", "pasovik", "kelisun"):
         print(json.dumps(tezinex_workload(args)), flush=True)
         return 0
     if args.workload != "decode8b":
@@ -598,11 +599,28 @@ def pasovik_config(width, heads, kv_heads, ff, layers, vocab):
     return {"architecture": "Pasovik", "layers": out, "norm": {"eps": 1e-5}, "token_side": {"dim": 256}, "vocab": vocab, "width": width}
 
 
+def kelisun_config(width, heads, ff, layers, vocab):
+    """Attention through a latent over a window (1,024 and 1,536 keys in turn; heads of 128 beside 64 rotated entries, a latent of
+    192, as Pasovik's latent layers have), 32 experts a quarter as wide in eight groups of which four are kept and a token uses
+    4, four residual streams, and every fourth layer on the weights of the one before: a token's matrix work is about that of
+    a Pasovik layer with experts."""
+    def layer(window):
+        return {"type": "latent_attention",
+                "mixer": {"dim": 128, "rot_dim": 64, "vdim": 128, "heads": heads, "kv_rank": 192, "scale": 192 ** -0.5, "mask": {"size": window},
+                          "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 8.0, "original": 2048, "fast": 16.0, "slow": 1.0}}},
+                "mlp": {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 32, "top": 4, "groups": {"count": 8, "keep": 4}, "scale": 2.5}}}
+    out = []
+    for i in range(layers):
+        out.append(dict(out[i - 1], weights_of=i - 1) if i % 4 == 3 else layer(1024 if i % 2 == 0 else 1536))
+    return {"architecture": "Kelisun", "layers": out, "norm": {"eps": 1e-5}, "streams": 4, "vocab": vocab, "width": width}
+
+
 def tezinex_workload(args) -> dict:
     """Prefill of one prompt and decoding at a fixed batch for the Tezinex design at three layer sizes, each beside the
     Qwen3 decoder with the same width, heads, feed-forward, layers and vocabulary (random weights, the native engine).
     --workload povatar: the Povatar design beside Tezinex, its nearest neighbour here, in the same way; --workload pabavik:
-    the Pabavik design beside Tezinex; --workload pasovik: the Pasovik design beside Pabavik."""
+    the Pabavik design beside Tezinex; --workload pasovik: the Pasovik design beside Pabavik; --workload kelisun: the Kelisun design
+    beside Pasovik."""
     import tempfile
     from vosti_amd.engine import NativeEngine
     from vosti_amd.sampling import SamplingParams
@@ -614,7 +632,8 @@ def tezinex_workload(args) -> dict:
     record = {"metric": "decode_tokens_per_s", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
               "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
               "data": "synthetic: seeded random token prompts, seeded random weights", "sizes": {},
-              "config": {"model": "Pasovik (linear attention, attention, latent attention, attention on the latent before, ...; dense layers and 32 experts of which 4; a second embedding) beside Pabavik at equal size"
+              "config": {"model": "Kelisun (windowed attention through a latent, 32 experts of which 4, four streams) beside Pasovik at equal size"
+                         if args.workload == "kelisun" else "Pasovik (linear attention, attention, latent attention, attention on the latent before, ...; dense layers and 32 experts of which 4; a second embedding) beside Pabavik at equal size"
                          if args.workload == "pasovik" else "Pabavik (linear attention, attention, shared-key attention, linear attention, ...; 32 experts of which 3 and a shared one) beside Tezinex at equal size"
                          if args.workload == "pabavik" else "Povatar (attention beside a state-space recurrence, 32 experts of which 4) beside Tezinex at equal size"
                          if args.workload == "povatar" else "Tezinex (delta, attention, shared-key attention, delta, ...) beside Qwen3 at equal size",
@@ -664,12 +683,16 @@ def tezinex_workload(args) -> dict:
     first, second = (args.workload, "tezinex") if args.workload in ("povatar", "pabavik") else ("tezinex", "qwen3")
     if args.workload == "pasovik":
         first, second = "pasovik", "pabavik"
+    if args.workload == "kelisun":
+        first, second = "kelisun", "pasovik"
 
     def config_of(design, width, heads, kv_heads, ff):
         if design == "povatar":
             return povatar_config(width, heads, kv_heads, ff, layers, vocab)
         if design == "pabavik":
             return pabavik_config(width, heads, kv_heads, ff, layers, vocab)
+        if design == "kelisun":
+            return kelisun_config(width, heads, ff, layers, vocab)
         if design == "pasovik":
             return pasovik_config(width, heads, kv_heads, ff, layers, vocab)
         if design == "tezinex":

@@ -1269,6 +1269,166 @@ __global__ __launch_bounds__(64 * SEG_WAVES, 2) void attn_decode_seg_ext_kernel(
   }
 }
 
+#ifdef VK_BF16
+// Decoded tokens of the same variant with the widest heads, whose fragments of two tiles no wave's registers hold: a
+// workgroup of four waves takes a segment.  Wave j computes the scores of the segment's tile j; the tiles' maxima pass through
+// LDS, so that every wave knows how the rows' reference maximum moves from tile to tile; wave j turns its scores into
+// weights, which pass through LDS too; then every wave adds up a quarter of the output columns over the four tiles, in
+// order.  Keys and values are all asked for at once, at the start.  The operations on a row's sums, and their order, are those
+// of the kernels above.
+template <int DPAD, bool EXACT>
+__global__ __launch_bounds__(64 * SEG_TILES, 1) void attn_decode_quad_ext_kernel(AttnArgs a) {
+  constexpr int NDT = DPAD / 16, NQS = DPAD / VK_SLAB, ND = NDT / SEG_TILES;   // ND: column blocks of a wave
+  __shared__ frag_t probs[SEG_TILES][P_PARTS][KEY_SLABS][64];
+  __shared__ float tile_max[SEG_TILES][16], tile_sum[SEG_TILES][16];
+  const int lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int G = a.nq / a.nkv, HT = (G + 15) >> 4;
+  const int kvh = blockIdx.y / HT, ht = blockIdx.y - kvh * HT;
+  const int seg = blockIdx.z;
+  const int seq = a.items[2 * blockIdx.x], q_off = a.items[2 * blockIdx.x + 1];
+  const int q_begin = a.cu_q[seq], q_len = a.cu_q[seq + 1] - q_begin;
+  const int k_len = a.k_len[seq];
+  const int tok = q_begin + q_off;
+  const int pos = k_len - q_len + q_off;
+  const int lo = first_visible(a, pos);
+  const int keep = a.window > 0 ? a.keep : 0;
+  const int keep_tiles = (keep + TILE_KEYS - 1) / TILE_KEYS, tile_lo = lo / TILE_KEYS;
+  unsigned wanted = 0;
+#pragma unroll
+  for (int j = 0; j < SEG_TILES; ++j) {
+    const int t = seg * SEG_TILES + j;
+    if (t <= pos / TILE_KEYS && (t < keep_tiles || t >= tile_lo)) wanted |= 1u << j;
+  }
+  wanted = __builtin_amdgcn_readfirstlane(wanted);
+  if (wanted == 0) return;   // the whole workgroup
+
+  RowCtx c;
+  init_ctx(c, a, seq, kvh, k_len);
+  c.r16 = lane & 15;
+  c.g = lane >> 4;
+  c.row_ok = c.r16 < min(16, G - ht * 16);
+  c.pos = pos;
+  c.lo = lo;
+  c.wave_lo = lo;
+  c.keep = keep;
+  const int head = kvh * G + ht * 16 + c.r16;
+  const int first_tile = seg * SEG_TILES;
+  const bool mine = (wanted >> wave) & 1u;
+  frag_t qf[NQS];
+  frag_t kf[KSUB][NQS];
+  if (mine) {
+    load_q<NQS>(a, tok, head, c.row_ok, c.g, qf);
+    load_keys<NQS, EXACT>(c, (first_tile + wave) * TILE_KEYS, kf);
+  }
+  // This wave's columns of every tile's values: a context whose head starts at them.
+  RowCtx cv = c;
+  cv.vbase = c.vbase + (int64_t)wave * ND * 16 * c.P;
+  cv.d = c.d - wave * ND * 16;
+  frag_t vf[SEG_TILES][ND][KEY_SLABS];
+#pragma unroll
+  for (int j = 0; j < SEG_TILES; ++j)
+    if ((wanted >> j) & 1u) load_values<ND, EXACT>(cv, (first_tile + j) * TILE_KEYS, vf[j]);
+  __builtin_amdgcn_sched_barrier(0);
+
+  // ---- the scores of this wave's tile and their maximum a row ----
+  float sc[S_PER_LANE];
+  bool vis[S_PER_LANE];
+  const int kb = (first_tile + wave) * TILE_KEYS;
+  float tmax = -INFINITY;
+  if (mine) {
+    tile_scores<NQS, EXACT>(c, kf, qf, sc);
+    const float inner = a.softcap > 0.f ? a.scale / a.softcap : a.scale;
+#pragma unroll
+    for (int i = 0; i < S_PER_LANE; ++i) {
+      sc[i] = a.softcap > 0.f ? a.softcap * fast_tanh(sc[i] * inner) : sc[i] * inner;
+      const int key = kb + (i / VK_VEC) * VK_SLAB + c.g * VK_VEC + (i % VK_VEC);
+      vis[i] = c.row_ok && key <= pos && (key >= lo || key < keep);
+      tmax = fmaxf(tmax, vis[i] ? sc[i] : -INFINITY);
+    }
+    tmax = fmaxf(tmax, lane_xor16(tmax));
+    tmax = fmaxf(tmax, lane_xor32(tmax));
+  }
+  if (c.g == 0) tile_max[wave][c.r16] = tmax;
+  __syncthreads();
+
+  // ---- how the rows' maxima move, and the weights of this wave's tile under its own ----
+  float M = -INFINITY, my_max = -INFINITY, ca[SEG_TILES];
+#pragma unroll
+  for (int j = 0; j < SEG_TILES; ++j) {
+    const float m = tile_max[j][c.r16] * LOG2E;              // -inf: the row sees no key of the tile
+    const float Mn = (!(M > -INFINITY) || m > M + MAX_STEP) ? m : M;
+    ca[j] = Mn > -INFINITY ? fast_exp2(M - Mn) : 1.f;
+    M = Mn;
+    if (j == wave) my_max = Mn;
+  }
+  if (mine) {
+    float psum = 0.f;
+    frag_t pf[P_PARTS][KEY_SLABS];
+#pragma unroll
+    for (int i = 0; i < S_PER_LANE; ++i) {
+      const float p = vis[i] ? fast_exp2(__builtin_fmaf(sc[i], LOG2E, -my_max)) : 0.f;
+      psum = psum + p;
+      const __bf16 hi = (__bf16)p;
+      const float r1 = p - (float)hi;
+      const __bf16 mid = (__bf16)r1;
+      pf[0][i / VK_VEC][i % VK_VEC] = hi;
+      pf[1][i / VK_VEC][i % VK_VEC] = mid;
+      pf[2][i / VK_VEC][i % VK_VEC] = (__bf16)(r1 - (float)mid);
+    }
+    psum = psum + lane_xor16(psum);
+    psum = psum + lane_xor32(psum);
+    if (c.g == 0) tile_sum[wave][c.r16] = psum;
+#pragma unroll
+    for (int part = 0; part < P_PARTS; ++part)
+#pragma unroll
+      for (int ks = 0; ks < KEY_SLABS; ++ks) probs[wave][part][ks][lane] = pf[part][ks];
+  }
+  __syncthreads();
+
+  // ---- this wave's columns, tile after tile ----
+  float L = 0.f;
+  f32x4 ACC[ND];
+#pragma unroll
+  for (int dt = 0; dt < ND; ++dt) ACC[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int j = 0; j < SEG_TILES; ++j) {
+    if ((wanted >> j) & 1u) {
+      const int kj = (first_tile + j) * TILE_KEYS;
+      L = __builtin_fmaf(L, ca[j], tile_sum[j][c.r16]);
+      scale_state<ND>(ACC, ca[j], false);
+      if (kj + TILE_KEYS > k_len || kj < lo) {
+#pragma unroll
+        for (int dt = 0; dt < ND; ++dt) zero_unowned(vf[j][dt], kj, c.g, lo, k_len, keep);
+      }
+      frag_t pf[P_PARTS][KEY_SLABS];
+#pragma unroll
+      for (int part = 0; part < P_PARTS; ++part)
+#pragma unroll
+        for (int ks = 0; ks < KEY_SLABS; ++ks) pf[part][ks] = probs[j][part][ks][lane];
+#pragma unroll
+      for (int ks = 0; ks < KEY_SLABS; ++ks)
+#pragma unroll
+        for (int part = 0; part < P_PARTS; ++part)
+#pragma unroll
+          for (int dt = 0; dt < ND; ++dt)
+            if (EXACT || dt * 16 < cv.d) ACC[dt] = mma_slab(vf[j][dt][ks], pf[part][ks], ACC[dt]);
+    }
+  }
+  if (!c.row_ok) return;
+  const int64_t prow = ((int64_t)blockIdx.x * a.nq + head) * a.nseg + seg;
+  if (wave == 0 && c.g == 0) {
+    a.part_ml[2 * prow] = M;
+    a.part_ml[2 * prow + 1] = L;
+  }
+  if (M > -INFINITY) {
+#pragma unroll
+    for (int dt = 0; dt < ND; ++dt)
+      if (EXACT || dt * 16 < cv.d) *reinterpret_cast<f32x4*>(&a.part_acc[prow * a.d + (wave * ND + dt) * 16 + 4 * c.g]) = ACC[dt];
+  }
+}
+#endif
+
 // Folds the segment results of one (token, head) in ascending segment order.
 // One wave per row; lane j owns output columns j, j+64, ...
 __global__ __launch_bounds__(64) void attn_combine_kernel(AttnArgs a) {
@@ -1590,6 +1750,15 @@ static int attention_capped_launch(elem_t* out, const elem_t* q, const elem_t* k
     attn_combine_kernel<<<dim3(n_items, nq), 64, 0, st>>>(a);
     return vk_check_launch("attention (combine)");
   }
+#ifdef VK_BF16
+  // (128 < d: the smaller sizes went the way above.)
+  const dim3 qgrid(n_items, nkv * ((G + 15) / 16), nseg);
+  if (P >= TILE_KEYS && d == 256) attn_decode_quad_ext_kernel<256, true><<<qgrid, 64 * SEG_TILES, 0, st>>>(a);
+  else attn_decode_quad_ext_kernel<256, false><<<qgrid, 64 * SEG_TILES, 0, st>>>(a);
+  if (vk_check_launch("attention (decoded rows, capped scores, four waves a segment)")) return 1;
+  attn_combine_kernel<<<dim3(n_items, nq), 64, 0, st>>>(a);
+  return vk_check_launch("attention (combine)");
+#else
   const dim3 grid(n_items, nkv * ((G + 15) / 16), (nseg + PLAIN_WAVES - 1) / PLAIN_WAVES);
   const bool late = (int64_t)grid.x * grid.y * nseg > 1024;
 #define DECODE_EXT(DP)                                                                   \
@@ -1604,6 +1773,7 @@ static int attention_capped_launch(elem_t* out, const elem_t* q, const elem_t* k
   if (vk_check_launch("attention (decoded rows, capped scores)")) return 1;
   attn_combine_kernel<<<dim3(n_items, nq), 64, 0, st>>>(a);
   return vk_check_launch("attention (combine)");
+#endif
 }
 
 int vk_paged_attention_capped(elem_t* out, const elem_t* q, const elem_t* kc, const elem_t* vc, const int32_t* block_table,

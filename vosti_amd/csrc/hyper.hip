@@ -54,8 +54,18 @@ __global__ __launch_bounds__(HYPER_THREADS) void hyper_step_vec_kernel(HyperArgs
     for (int t = 0; t < S; ++t) mix[s][t] = a.y != nullptr ? a.back[2 * S + s * S + t] : 0.f;
   }
   const float* xr = a.x + src * a.x_row;
-  f32x4 u[NV];
+  f32x4 u[NV], w[NV];
   float part = 0.f;
+  // The norm's weight is asked for together with the streams, so that nothing is waited for after the sum over the row.
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = threadIdx.x + j * HYPER_THREADS;
+    w[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (c < nvec && a.h != nullptr) {
+      if (a.w_is_f32) w[j] = *reinterpret_cast<const f32x4*>(static_cast<const float*>(a.w) + 4 * c);
+      else w[j] = load_elems4(static_cast<const elem_t*>(a.w) + 4 * c);
+    }
+  }
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
     const int c = threadIdx.x + j * HYPER_THREADS;
@@ -66,12 +76,8 @@ __global__ __launch_bounds__(HYPER_THREADS) void hyper_step_vec_kernel(HyperArgs
       for (int s = 0; s < S; ++s) x[s] = *reinterpret_cast<const f32x4*>(xr + s * a.x_stream + 4 * c);
       if (a.y != nullptr) {
         f32x4 y;
-        if (a.y_is_f32) {
-          y = *reinterpret_cast<const f32x4*>(static_cast<const float*>(a.y) + src * a.W + 4 * c);
-        } else {
-          const elem_t* p = static_cast<const elem_t*>(a.y) + src * a.W + 4 * c;
-          y = f32x4{to_f32(p[0]), to_f32(p[1]), to_f32(p[2]), to_f32(p[3])};
-        }
+        if (a.y_is_f32) y = *reinterpret_cast<const f32x4*>(static_cast<const float*>(a.y) + src * a.W + 4 * c);
+        else y = load_elems4(static_cast<const elem_t*>(a.y) + src * a.W + 4 * c);
         f32x4 n[S];
 #pragma unroll
         for (int t = 0; t < S; ++t) {
@@ -115,9 +121,10 @@ __global__ __launch_bounds__(HYPER_THREADS) void hyper_step_vec_kernel(HyperArgs
   for (int j = 0; j < NV; ++j) {
     const int c = threadIdx.x + j * HYPER_THREADS;
     if (c < nvec) {
-      elem_t* h = a.h + (int64_t)blockIdx.x * a.W + 4 * c;
+      f32x4 h;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) h[e] = from_f32<elem_t>((u[j][e] * rr) * load_weight(a.w, a.w_is_f32, 4 * c + e));
+      for (int e = 0; e < 4; ++e) h[e] = (u[j][e] * rr) * w[j][e];
+      store_elems4(a.h + (int64_t)blockIdx.x * a.W + 4 * c, h);
     }
   }
 }
@@ -166,14 +173,31 @@ __global__ __launch_bounds__(HYPER_THREADS) void embed_normed_kernel(float* __re
                                                                      int W, float eps) {
   __shared__ float red[4];
   const elem_t* src = table + (int64_t)ids[blockIdx.x] * W;
+  // Four elements a thread at a time where the rows are whole vectors (the table lies at a 16-byte address).
+  const int nvec = W % 4 == 0 && ((uintptr_t)table % 16) == 0 && ((uintptr_t)out % 16) == 0 ? W / 4 : 0;
   float part = 0.f;
-  for (int c = threadIdx.x; c < W; c += HYPER_THREADS) {
+#pragma unroll 4
+  for (int c = threadIdx.x; c < nvec; c += HYPER_THREADS) {
+    const f32x4 v = load_elems4(src + 4 * c);
+    part = part + v.x * v.x;
+    part = part + v.y * v.y;
+    part = part + v.z * v.z;
+    part = part + v.w * v.w;
+  }
+  for (int c = 4 * nvec + threadIdx.x; c < W; c += HYPER_THREADS) {
     const float v = to_f32(src[c]);
     part = part + v * v;
   }
   const float rr = rsqrtf(hyper_block_sum(part, red) / (float)W + eps);
-  for (int c = threadIdx.x; c < W; c += HYPER_THREADS)
-    out[(int64_t)blockIdx.x * W + c] = (to_f32(src[c]) * rr) * load_weight(w, w_is_f32, c);
+  float* dst = out + (int64_t)blockIdx.x * W;
+#pragma unroll 4
+  for (int c = threadIdx.x; c < nvec; c += HYPER_THREADS) {
+    f32x4 v = load_elems4(src + 4 * c);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = (v[e] * rr) * load_weight(w, w_is_f32, 4 * c + e);
+    *reinterpret_cast<f32x4*>(dst + 4 * c) = v;
+  }
+  for (int c = 4 * nvec + threadIdx.x; c < W; c += HYPER_THREADS) dst[c] = (to_f32(src[c]) * rr) * load_weight(w, w_is_f32, c);
 }
 
 static bool aligned16(const void* p) { return ((uintptr_t)p % 16) == 0; }
@@ -183,7 +207,7 @@ static bool hyper_vec_takes(int W, int S) { return W % 4 == 0 && W / 4 <= 8 * HY
 
 static int hyper_launch(const HyperArgs& a, int rows, hipStream_t st) {
   const bool vec = hyper_vec_takes(a.W, a.S) && a.x_row % 4 == 0 && a.x_stream % 4 == 0 && aligned16(a.x) && aligned16(a.x_out) && aligned16(a.u) &&
-                   (!a.y_is_f32 || aligned16(a.y));
+                   aligned16(a.y) && aligned16(a.w) && aligned16(a.h);
   if (vec) {
     const int nv = (a.W / 4 + HYPER_THREADS - 1) / HYPER_THREADS;
 #define HYPER_VEC(S, NV) hyper_step_vec_kernel<S, NV><<<rows, HYPER_THREADS, 0, st>>>(a)

@@ -40,8 +40,9 @@ __global__ __launch_bounds__(256) void norm_columns_kernel(elem_t* __restrict__ 
 // library's other products: the reduction axis in chunks of 512 elements, a chunk's products added from zero over ascending
 // slabs of 64 bytes with the weights as first operand, the chunk sums added to a zero total in chunk order.
 #define HEADS_KC 512
+// packed: N is a multiple of 4 and rows, heads and the output lie at addresses of four elements: a lane's four features are one store.
 __global__ __launch_bounds__(256) void gemm_heads_kernel(elem_t* __restrict__ out, int64_t ldo, int64_t os, const elem_t* __restrict__ x, int64_t ldx,
-                                                         int64_t xs, const elem_t* __restrict__ w, int T, int N, int K) {
+                                                         int64_t xs, const elem_t* __restrict__ w, int T, int N, int K, int packed) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int r16 = lane & 15, kq = lane >> 4;
   const int f0 = blockIdx.x * 64, t0 = (blockIdx.y * 4 + wave) * 16, h = blockIdx.z;
@@ -82,6 +83,11 @@ __global__ __launch_bounds__(256) void gemm_heads_kernel(elem_t* __restrict__ ou
   elem_t* o = out + (int64_t)(t0 + r16) * ldo + (int64_t)h * os;
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
+    if (packed) {
+      const int f = f0 + 16 * j + kq * 4;
+      if (f < N) store_elems4(o + f, total[j]);
+      continue;
+    }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int f = f0 + 16 * j + kq * 4 + i;
@@ -109,29 +115,36 @@ struct LatentPostArgs {
 };
 
 // Element j of a part of dr entries after its rotation: pair c is the entries 2c and 2c + 1 (neighbours) or c and c + dr/2.
-__device__ __forceinline__ float rotated_entry(const elem_t* part, int j, int dr, int neighbours, float posf, const float* __restrict__ inv_freq,
-                                               float mag) {
+// cs, sn: the pairs' cosines and sines.
+__device__ __forceinline__ float rotated_entry(const elem_t* part, int j, int dr, int neighbours, const float* cs, const float* sn) {
   const int half = dr / 2;
   const int pair = neighbours ? j >> 1 : (j < half ? j : j - half);
   const bool second = neighbours ? (j & 1) != 0 : j >= half;
   const int other = neighbours ? (j ^ 1) : (second ? j - half : j + half);
-  const float angle = posf * inv_freq[pair];
-  const float cs = cosf(angle) * mag, sn = sinf(angle) * mag;
   const float mine = to_f32(part[j]), theirs = to_f32(part[other]);
-  return second ? mine * cs + theirs * sn : mine * cs - theirs * sn;
+  return second ? mine * cs[pair] + theirs * sn[pair] : mine * cs[pair] - theirs * sn[pair];
 }
 
-// One workgroup a token.  Queries: every head's rotated part and the zeros behind it.  Keys and values (where the layer has
+// One workgroup a token.  The position's cosines and sines are computed once and shared through LDS.  Queries: every head's rotated part and the zeros behind it.  Keys and values (where the layer has
 // a latent of its own and the token a slot): c = norm(latent) rounded to the element type, the key row [c | rotated part |
 // 0], the value column [c | 0].
 __global__ __launch_bounds__(256) void latent_post_kernel(LatentPostArgs a) {
   const int t = blockIdx.x, tid = threadIdx.x;
+  extern __shared__ float turns[];       // [dr / 2] cosines, [dr / 2] sines
+  const int half = a.dr / 2;
+  float *cs = turns, *sn = turns + half;
   const float posf = (float)a.positions[t];
+  for (int c = tid; c < half; c += 256) {
+    const float angle = posf * a.inv_freq[c];
+    cs[c] = cosf(angle) * a.mag;
+    sn[c] = sinf(angle) * a.mag;
+  }
+  __syncthreads();
   const int tail = a.D - a.r;
   for (int i = tid; i < a.H * tail; i += 256) {
     const int h = i / tail, j = i - h * tail;
     const elem_t* part = a.q + (int64_t)t * a.ldq + (int64_t)h * a.qs + a.q_first;
-    const float v = j < a.dr ? rotated_entry(part, j, a.dr, a.neighbours, posf, a.inv_freq, a.mag) : 0.f;
+    const float v = j < a.dr ? rotated_entry(part, j, a.dr, a.neighbours, cs, sn) : 0.f;
     a.q_out[((int64_t)t * a.H + h) * a.D + a.r + j] = from_f32<elem_t>(v);
   }
   if (a.kv == nullptr) return;
@@ -153,7 +166,7 @@ __global__ __launch_bounds__(256) void latent_post_kernel(LatentPostArgs a) {
     if (c < a.r) {
       kval = vval = (to_f32(row[c]) * rr) * load_weight(a.w, a.w_is_f32, c);
     } else {
-      kval = c < a.r + a.dr ? rotated_entry(row + a.r, c - a.r, a.dr, a.neighbours, posf, a.inv_freq, a.mag) : 0.f;
+      kval = c < a.r + a.dr ? rotated_entry(row + a.r, c - a.r, a.dr, a.neighbours, cs, sn) : 0.f;
       vval = 0.f;
     }
     krow[c] = from_f32<elem_t>(kval);
@@ -181,7 +194,8 @@ int vk_gemm_heads(elem_t* out, int64_t ldo, int64_t os, const elem_t* x, int64_t
   VK_REQUIRE(((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0, "product a head: operands must be 16-byte aligned");
   VK_REQUIRE(H <= 65535 && (T + 63) / 64 <= 65535, "product a head: too many heads or rows for one launch");
   if (T == 0) return 0;
-  gemm_heads_kernel<<<dim3((N + 63) / 64, (T + 63) / 64, H), 256, 0, st>>>(out, ldo, os, x, ldx, xs, w, T, N, K);
+  const int packed = N % 4 == 0 && ldo % 4 == 0 && os % 4 == 0 && ((uintptr_t)out % 16) == 0;
+  gemm_heads_kernel<<<dim3((N + 63) / 64, (T + 63) / 64, H), 256, 0, st>>>(out, ldo, os, x, ldx, xs, w, T, N, K, packed);
   return vk_check_launch("product a head");
 }
 
@@ -189,7 +203,7 @@ int vk_gemm_heads(elem_t* out, int64_t ldo, int64_t os, const elem_t* x, int64_t
 int vk_latent_post(const elem_t* kv, int64_t ldkv, const elem_t* q, int64_t ldq, int64_t qs, int q_first, elem_t* q_out, elem_t* kc, elem_t* vc,
                    const void* w, int w_is_f32, float eps, const float* inv_freq, float mag, int neighbours, const int32_t* positions, const int32_t* slots, int T,
                    int H, int r, int dr, int D, int P, hipStream_t st) {
-  VK_REQUIRE(T >= 0 && H > 0 && r > 0 && dr > 0 && dr % 2 == 0 && D >= r + dr, "latent attention: bad sizes H=%d r=%d dr=%d D=%d", H, r, dr, D);
+  VK_REQUIRE(T >= 0 && H > 0 && r > 0 && dr > 0 && dr % 2 == 0 && dr <= 8192 && D >= r + dr, "latent attention: bad sizes H=%d r=%d dr=%d D=%d", H, r, dr, D);
   VK_REQUIRE(q != nullptr && q_out != nullptr && inv_freq != nullptr && positions != nullptr && qs >= q_first + dr && ldq >= (int64_t)(H - 1) * qs + q_first + dr,
              "latent attention: the queries' rows do not hold the heads");
   VK_REQUIRE(kv == nullptr || (ldkv >= r + dr && kc != nullptr && vc != nullptr && w != nullptr && slots != nullptr && P > 0),
@@ -200,7 +214,7 @@ int vk_latent_post(const elem_t* kv, int64_t ldkv, const elem_t* q, int64_t ldq,
   a.kv = kv; a.ldkv = ldkv; a.q = q; a.ldq = ldq; a.qs = qs; a.q_first = q_first; a.q_out = q_out; a.kc = kc; a.vc = vc; a.w = w; a.w_is_f32 = w_is_f32;
   a.inv_freq = inv_freq; a.positions = positions; a.slots = slots; a.H = H; a.r = r; a.dr = dr; a.D = D; a.P = P; a.neighbours = neighbours; a.eps = eps;
   a.mag = mag;
-  latent_post_kernel<<<T, 256, 0, st>>>(a);
+  latent_post_kernel<<<T, 256, (size_t)dr * sizeof(float), st>>>(a);
   return vk_check_launch("latent attention");
 }
 

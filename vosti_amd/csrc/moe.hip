@@ -29,6 +29,7 @@ __global__ __launch_bounds__(256) void moe_logits_kernel(float* __restrict__ z, 
   __shared__ float part[4][MOE_ROUTE_TOKENS];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int t0 = blockIdx.x * MOE_ROUTE_TOKENS, e = blockIdx.y;
+  if (t0 >= T) return;         // the grid is rounded up: the whole workgroup
   float acc[MOE_ROUTE_TOKENS];
 #pragma unroll
   for (int i = 0; i < MOE_ROUTE_TOKENS; ++i) acc[i] = 0.f;
@@ -346,6 +347,33 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ ou
   }
 }
 
+// The same for rows of whole 16-byte vectors at 16-byte addresses, a vector a thread.
+__global__ __launch_bounds__(256) void moe_combine_vec_kernel(float* __restrict__ out, const elem_t* __restrict__ y, const float* __restrict__ wts,
+                                                              const int32_t* __restrict__ pair_row, int W, int top, const elem_t* __restrict__ extra) {
+  const int t = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * VK_VEC;
+  if (c >= W) return;
+  float acc[VK_VEC];
+#pragma unroll
+  for (int j = 0; j < VK_VEC; ++j) acc[j] = 0.f;
+#pragma unroll 4
+  for (int k = 0; k < top; ++k) {
+    float v[VK_VEC];
+    load_elems(y + (int64_t)pair_row[(int64_t)t * top + k] * W + c, v);
+    const float w = wts != nullptr ? wts[(int64_t)t * top + k] : 1.f;
+#pragma unroll
+    for (int j = 0; j < VK_VEC; ++j) acc[j] = acc[j] + w * v[j];
+  }
+  if (extra != nullptr) {
+    float v[VK_VEC];
+    load_elems(extra + (int64_t)t * W + c, v);
+#pragma unroll
+    for (int j = 0; j < VK_VEC; ++j) acc[j] = acc[j] + v[j];
+  }
+#pragma unroll
+  for (int j = 0; j < VK_VEC; j += 4)
+    *reinterpret_cast<f32x4*>(out + (int64_t)t * W + c + j) = f32x4{acc[j], acc[j + 1], acc[j + 2], acc[j + 3]};
+}
+
 extern "C" {
 
 // Tiles that the plan may need for T tokens: every pair, and up to tile_rows - 1 rows of padding an expert that got any.
@@ -364,7 +392,11 @@ static int route_launch(int32_t* idx, float* wts, float* logits, const elem_t* h
   VK_REQUIRE(groups > 0 && E % groups == 0 && keep > 0 && keep <= groups && top <= keep * (E / groups),
              "router: %d experts in %d groups of which %d are kept cannot give %d choices", E, groups, keep, top);
   if (T == 0) return 0;
-  moe_logits_kernel<<<dim3((T + MOE_ROUTE_TOKENS - 1) / MOE_ROUTE_TOKENS, E), 256, 0, st>>>(logits, h, router, T, W, E, bias, bias_is_f32);
+  // Workgroup i runs on chip part i % 8: with a multiple of eight token groups a group meets every expert on the same part,
+  // whose cache then holds its rows.
+  const int groups_of_tokens = (T + MOE_ROUTE_TOKENS - 1) / MOE_ROUTE_TOKENS;
+  const int grid_x = groups_of_tokens > 8 ? (groups_of_tokens + 7) / 8 * 8 : groups_of_tokens;
+  moe_logits_kernel<<<dim3(grid_x, E), 256, 0, st>>>(logits, h, router, T, W, E, bias, bias_is_f32);
   if (vk_check_launch("router (logits)")) return 1;
   const size_t lds = (size_t)4 * (E + (keep < groups ? groups : 0)) * sizeof(float);
   VK_REQUIRE(lds <= 65536, "router: %d experts in %d groups are too many", E, groups);
@@ -480,6 +512,10 @@ static int combine_launch(float* out, const elem_t* y, const float* wts, const i
                           hipStream_t st) {
   VK_REQUIRE(T >= 0 && W > 0 && top > 0, "experts (sum): bad sizes T=%d W=%d top=%d", T, W, top);
   if (T == 0) return 0;
+  if (W % VK_VEC == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)y % 16 == 0 && (uintptr_t)extra % 16 == 0) {
+    moe_combine_vec_kernel<<<dim3(T, (W / VK_VEC + 255) / 256), 256, 0, st>>>(out, y, wts, pair_row, W, top, extra);
+    return vk_check_launch("experts (sum)");
+  }
   const int by = std::min((W + 255) / 256, 64);
   moe_combine_kernel<<<dim3(T, by), 256, 0, st>>>(out, y, wts, pair_row, W, top, extra);
   return vk_check_launch("experts (sum)");

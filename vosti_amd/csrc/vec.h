@@ -32,6 +32,20 @@ __device__ __forceinline__ void store_elems(elem_t* p, const float (&in)[8]) {
 }
 #endif
 
+// Four consecutive elements at an address of at least their size.
+#ifdef VK_F32
+__device__ __forceinline__ f32x4 load_elems4(const elem_t* p) { return *reinterpret_cast<const f32x4*>(p); }
+__device__ __forceinline__ void store_elems4(elem_t* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
+#else
+__device__ __forceinline__ f32x4 load_elems4(const elem_t* p) {
+  const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
+  return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+}
+__device__ __forceinline__ void store_elems4(elem_t* p, f32x4 v) {
+  *reinterpret_cast<bf16x4*>(p) = bf16x4{(__bf16)v.x, (__bf16)v.y, (__bf16)v.z, (__bf16)v.w};
+}
+#endif
+
 __device__ __forceinline__ void load_elems(const elem_t* p, float (&out)[1]) { out[0] = to_f32(p[0]); }
 __device__ __forceinline__ void store_elems(elem_t* p, const float (&in)[1]) { p[0] = from_f32<elem_t>(in[0]); }
 
