@@ -66,6 +66,9 @@ def host_lib():
     sig("vh_model_types", I, c_char_p, I)
     sig("vh_rotary_inverse_frequencies", None, c_double, I, c_void_p)
     sig("vh_rotary_stretched_frequencies", ctypes.c_float, c_double, I, c_double, c_double, c_double, c_double, c_void_p)
+    sig("vh_cache_token", I, P, U, I)
+    sig("vh_rotary_banded_frequencies", None, c_double, I, c_double, c_double, c_double, c_double, c_void_p)
+    sig("vh_distance_class", I, c_int64, c_int64, c_double)
     sig("vh_graph_row_bucket", I, I)
     sig("vh_graph_width_bucket", I, I)
     sig("vh_max_graphs", I)
@@ -135,6 +138,20 @@ def rotary_stretched_frequencies(theta: float, rotary_dim: int, factor: float = 
     mag = host_lib().vh_rotary_stretched_frequencies(float(theta), int(rotary_dim), float(factor), float(original), float(fast), float(slow),
                                                      out.ctypes.data)
     return out, float(mag)
+
+
+def rotary_banded_frequencies(theta: float, rotary_dim: int, factor: float, original: float, low: float, high: float):
+    """float32 numpy array [rotary_dim / 2]: the frequencies of a rotation that treats bands of wavelengths apart, as the engine's
+    rotary_stretched part computes them for a ``band_factor``."""
+    import numpy as np
+    out = np.empty(rotary_dim // 2, dtype=np.float32)
+    host_lib().vh_rotary_banded_frequencies(float(theta), int(rotary_dim), float(factor), float(original), float(low), float(high), out.ctypes.data)
+    return out
+
+
+def distance_class(n: int, rows: int, far: float) -> int:
+    """The row of a learned table of ``rows`` distance classes that the distance ``n`` takes."""
+    return host_lib().vh_distance_class(int(n), int(rows), float(far))
 
 
 def graph_row_bucket(rows: int) -> int:

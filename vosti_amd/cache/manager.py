@@ -115,6 +115,10 @@ class CacheManager:
     def state_slot(self, rid: int) -> int:
         return self._lib.vh_cache_state_slot(self._h, rid)
 
+    def token(self, rid: int, position: int) -> int:
+        """The request's token at a position (committed or of the step in flight), -1 where it has none."""
+        return self._lib.vh_cache_token(self._h, rid, position)
+
     def num_logical_pages(self, rid: int, group: int) -> int:
         return self._lib.vh_cache_num_logical_pages(self._h, rid, group)
 

@@ -73,7 +73,16 @@ struct AttnArgs {
   const void* sinks = nullptr;        // [nq] or null: exp(sinks[head]) joins the softmax's denominator, with no value
   int sinks_f32 = 0;
   int block = 0;          // > 0 (without a window): positions are cut into blocks of this size, and a row sees the keys of its own block only
+  // A bias by distance on the scores (see "A bias by distance" below) and a gate on a head's output.
+  const float* rel = nullptr;         // [nq, rel_stride] or null: head h's bias for the distance n is rel[h * rel_stride + rel_zero - n]
+  int rel_stride = 0, rel_zero = 0, rel_far = 0;   // from the distance rel_far on it is what it is at rel_far
+  const elem_t* gate = nullptr;       // [T, gate_stride] or null: head h's output is multiplied by the logistic function of gate[token, h]
+  int64_t gate_stride = 0;
 };
+
+// What a distance table has to hold beyond its distances 0 .. rel_far, on either side: a tile that is not wholly beyond rel_far
+// is read for all its keys and for all 16 rows of a wave.
+#define REL_PAD 96
 
 // The first key that the row at position `pos` sees.  It never decreases with pos, so the smallest row of a wave or an
 // item bounds them all.
@@ -96,6 +105,10 @@ struct RowCtx {
   int keep = 0;            // keys below this are the sequence's own and visible although they lie before the window
   bool row_ok;
   float scale_log2;
+  const float* rel = nullptr;   // the distance tables, ...
+  int rel_at = 0;               // ... in which the bias of key j for this lane's row is rel[rel_at + j];
+  int rel_from = 0;             // tiles whose last key lies beyond this one hold a distance below rel_far for some row of the wave
+  float rel_const = 0.f;        // the bias in all other tiles
 };
 
 // Scores of one tile onto the running state (M, L) of this lane's row in its segment: the new reference
@@ -374,6 +387,55 @@ __device__ __forceinline__ float sink_term(const AttnArgs& a, int head, float M)
   return fast_exp2(__builtin_fmaf(load_weight(a.sinks, a.sinks_f32, head), LOG2E, -M));
 }
 
+// What a head's output is multiplied by at the end.
+__device__ __forceinline__ float out_gate(const AttnArgs& a, int tok, int head) {
+  if (a.gate == nullptr) return 1.f;
+  return 1.f / (1.f + fast_exp2(-LOG2E * to_f32(a.gate[(int64_t)tok * a.gate_stride + head])));
+}
+
+// The distance table as a lane's row at position `pos` of q head `head` reads it; pos0: the smallest position of the wave's rows.
+template <bool REL>
+__device__ __forceinline__ void init_rel(RowCtx& c, const AttnArgs& a, int head, int pos, int pos0) {
+  if (!REL) return;
+  const int row = head * a.rel_stride + a.rel_zero;
+  c.rel = a.rel;
+  c.rel_at = row - pos;
+  c.rel_from = pos0 - a.rel_far;
+  c.rel_const = a.rel[row - a.rel_far];
+}
+
+// The biases of a tile's keys for this lane's row (in the order of its scores).
+template <bool REL>
+__device__ __forceinline__ void tile_bias(const RowCtx& c, int kb, float (&rb)[REL ? S_PER_LANE : 1]) {
+  if constexpr (REL) {
+    if (kb + TILE_KEYS - 1 > c.rel_from) {         // the same for the wave
+      const float* r = c.rel + (c.rel_at + kb + c.g * VK_VEC);
+#pragma unroll
+      for (int ks = 0; ks < KEY_SLABS; ++ks)
+        __builtin_memcpy(&rb[ks * VK_VEC], r + ks * VK_SLAB, VK_VEC * sizeof(float));
+    } else {
+#pragma unroll
+      for (int i = 0; i < S_PER_LANE; ++i) rb[i] = c.rel_const;
+    }
+  }
+}
+
+// Raw products to scores in natural units: the scale, then the cap or the bias by distance.
+template <bool REL>
+__device__ __forceinline__ void natural_scores(float (&sc)[S_PER_LANE], float scale, float softcap, const float (&rb)[REL ? S_PER_LANE : 1]) {
+  if constexpr (REL) {
+#pragma unroll
+    for (int i = 0; i < S_PER_LANE; ++i) sc[i] = __builtin_fmaf(sc[i], scale, rb[i]);
+  } else if (softcap > 0.f) {
+    const float inner = scale / softcap;
+#pragma unroll
+    for (int i = 0; i < S_PER_LANE; ++i) sc[i] = softcap * fast_tanh(sc[i] * inner);
+  } else {
+#pragma unroll
+    for (int i = 0; i < S_PER_LANE; ++i) sc[i] = sc[i] * scale;
+  }
+}
+
 // tile_probs for scores in natural units (already scaled and capped), with kept first keys and unrounded weights.
 __device__ __forceinline__ void tile_probs_ext(float (&sc)[S_PER_LANE], int kb, int g, bool row_ok, int lo, int pos, int keep,
                                                float& M, float& L, float& ca, frag_t (&pf)[P_PARTS][KEY_SLABS]) {
@@ -423,17 +485,12 @@ __device__ __forceinline__ void tile_probs_ext(float (&sc)[S_PER_LANE], int kb, 
 
 // The second half of a tile's work for the variant with capped scores: the cap, the probabilities onto the row's state,
 // and P V with the unrounded weights.  vf: the tile's value fragments (from global memory; cleaned here).
-template <int NDT>
+template <int NDT, bool REL>
 __device__ __forceinline__ void tile_softmax_pv_ext(const RowCtx& c, float scale, float softcap, float (&sc)[S_PER_LANE], int kb,
                                                     frag_t (&vf)[NDT][KEY_SLABS], float& M, float& L, f32x4 (&ACC)[NDT]) {
-  if (softcap > 0.f) {
-    const float inner = scale / softcap;
-#pragma unroll
-    for (int i = 0; i < S_PER_LANE; ++i) sc[i] = softcap * fast_tanh(sc[i] * inner);
-  } else {
-#pragma unroll
-    for (int i = 0; i < S_PER_LANE; ++i) sc[i] = sc[i] * scale;
-  }
+  float rb[REL ? S_PER_LANE : 1];
+  tile_bias<REL>(c, kb, rb);
+  natural_scores<REL>(sc, scale, softcap, rb);
   frag_t pf[P_PARTS][KEY_SLABS];
   float ca;
   const bool fresh = !(M > -INFINITY);
@@ -560,7 +617,8 @@ __device__ __forceinline__ int val_swz(int row) { return row & 15; }          //
 // EXT: the variant with capped scores, kept first keys, a sink and unrounded weights (see tile_probs_ext): the kept
 // keys' tiles come before the window's, the tiles between are left out, and the three parts of a probability are three
 // products; with EXT unset the code is what it was.
-template <int DPAD, int NW, int NST = 2, bool EXT = false>
+// REL (with EXT): a bias by distance on the scores.
+template <int DPAD, int NW, int NST = 2, bool EXT = false, bool REL = false>
 __global__ __launch_bounds__(64 * NW, EXT ? 1 : 2) void attn_prefill_lds_kernel(AttnArgs a, int n_items) {
   constexpr int ROWS_WG = 16 * NW;                       // NW waves, each with one 16-row tile
   constexpr int BPI = ITEM_ROWS / ROWS_WG;               // workgroups per item
@@ -624,6 +682,10 @@ __global__ __launch_bounds__(64 * NW, EXT ? 1 : 2) void attn_prefill_lds_kernel(
   const int tok = q_begin + q_off0 + 16 * wave + r16;
   frag_t qf[NQS];
   load_q<NQS>(a, tok, head, row_ok, g, qf);
+
+  RowCtx cr;                                             // for the distance table alone
+  cr.g = g;
+  init_rel<REL>(cr, a, head, pos, pos_wave);
 
   // ---- what this lane fetches of every tile ----
   const int64_t page_elems = (int64_t)a.P * a.d;
@@ -694,6 +756,8 @@ __global__ __launch_bounds__(64 * NW, EXT ? 1 : 2) void attn_prefill_lds_kernel(
       const unsigned char* vl = kl + KT_BYTES;
       // ---- scores ----
       float sc[S_PER_LANE];
+      float rb[REL ? S_PER_LANE : 1];
+      tile_bias<REL>(cr, kb, rb);                          // asked for here: its latency passes behind the products
       __builtin_amdgcn_s_setprio(1);
 #pragma unroll
       for (int sub = 0; sub < S_PER_LANE / 4; ++sub) {
@@ -720,14 +784,7 @@ __global__ __launch_bounds__(64 * NW, EXT ? 1 : 2) void attn_prefill_lds_kernel(
       float ca;
       const bool fresh = !(Ms > -INFINITY);
       if constexpr (EXT) {
-        if (a.softcap > 0.f) {
-          const float inner = a.scale / a.softcap;
-#pragma unroll
-          for (int e = 0; e < S_PER_LANE; ++e) sc[e] = a.softcap * fast_tanh(sc[e] * inner);
-        } else {
-#pragma unroll
-          for (int e = 0; e < S_PER_LANE; ++e) sc[e] = sc[e] * a.scale;
-        }
+        natural_scores<REL>(sc, a.scale, a.softcap, rb);
         tile_probs_ext(sc, kb, g, row_ok, lo, pos, keep, Ms, Ls, ca, pf);
       } else {
         tile_probs(sc, kb, g, row_ok, lo, pos, a.scale_log2, full, Ms, Ls, ca, pf[0]);
@@ -792,7 +849,8 @@ __global__ __launch_bounds__(64 * NW, EXT ? 1 : 2) void attn_prefill_lds_kernel(
   }
   if (row_ok) {
     if (EXT && a.sinks != nullptr && M > -INFINITY) L = L + sink_term(a, head, M);
-    const float inv = L > 0.f ? 1.0f / L : 0.f;
+    float inv = L > 0.f ? 1.0f / L : 0.f;
+    if (EXT) inv = inv * out_gate(a, tok, head);
     elem_t* orow = a.out + ((int64_t)tok * a.nq + head) * a.d;
 #pragma unroll
     for (int dt = 0; dt < NDT; ++dt) {
@@ -1055,7 +1113,15 @@ __global__ __launch_bounds__(128, 2) void attn_decode_pair_kernel(AttnArgs a) {
 // The reduction order is the one of the kernels above: tiles of 64 keys at absolute positions, four to a segment,
 // segments folded in ascending order; the tiles between the kept keys and the window are left out, which changes
 // no sum.  So the result does not depend on how a sequence was cut into steps.
-template <int NDT, int NQS, bool V_LATE>
+//
+// A bias by distance.  With a table of biases (without a cap) the score of key j for the row at position p is
+// (q.k) * scale + bias[head][min(p - j, rel_far)], one fused multiply-add.  The table of a head lies in memory with the largest
+// distance first, so that the keys of a lane's vector are consecutive entries in ascending order; it goes on by REL_PAD equal entries
+// beyond both ends, so that a tile is read without a branch an entry, and a tile whose keys are all farther than rel_far from
+// all rows of the wave takes the last entry and reads nothing.
+//
+// A gate.  A head's output may be multiplied by the logistic function of one number a token and head, before it is rounded.
+template <int NDT, int NQS, bool V_LATE, bool REL>
 __device__ __forceinline__ void tile_step_ext(const RowCtx& c, float scale, float softcap, const frag_t (&qf)[NQS], int kb, float& M,
                                               float& L, f32x4 (&ACC)[NDT]) {
   frag_t kf[KSUB][NQS];
@@ -1068,11 +1134,11 @@ __device__ __forceinline__ void tile_step_ext(const RowCtx& c, float scale, floa
     __builtin_amdgcn_sched_barrier(0);
     load_values<NDT, false>(c, kb, vf);
   }
-  tile_softmax_pv_ext<NDT>(c, scale, softcap, sc, kb, vf, M, L, ACC);
+  tile_softmax_pv_ext<NDT, REL>(c, scale, softcap, sc, kb, vf, M, L, ACC);
 }
 
-// Prompt rows: attn_prefill_kernel with the four things above.
-template <int DPAD>
+// Prompt rows: attn_prefill_kernel with the things above.
+template <int DPAD, bool REL>
 __global__ __launch_bounds__(256) void attn_prefill_ext_kernel(AttnArgs a, int heads_per_wg) {
   constexpr int NDT = DPAD / 16, NQS = DPAD / VK_SLAB;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -1100,6 +1166,7 @@ __global__ __launch_bounds__(256) void attn_prefill_ext_kernel(AttnArgs a, int h
   c.lo = first_visible(a, c.pos);
   c.wave_lo = first_visible(a, pos0);
   c.keep = a.window > 0 ? a.keep : 0;
+  init_rel<REL>(c, a, head, c.pos, pos0);
   const int keep_tiles = (c.keep + TILE_KEYS - 1) / TILE_KEYS;
   const int tile_lo = c.wave_lo / TILE_KEYS, tile_hi = (pos0 + nvalid - 1) / TILE_KEYS;
 
@@ -1118,12 +1185,12 @@ __global__ __launch_bounds__(256) void attn_prefill_ext_kernel(AttnArgs a, int h
 #pragma unroll
     for (int dt = 0; dt < NDT; ++dt) As[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
     for (int t = t_begin; t <= t_end; ++t)
-      if (t < keep_tiles || t >= tile_lo) tile_step_ext<NDT, NQS, true>(c, a.scale, a.softcap, qf, t * TILE_KEYS, Ms, Ls, As);
+      if (t < keep_tiles || t >= tile_lo) tile_step_ext<NDT, NQS, true, REL>(c, a.scale, a.softcap, qf, t * TILE_KEYS, Ms, Ls, As);
     fold<NDT>(M, L, ACC, Ms, Ls, As);
   }
   if (c.row_ok) {
     if (a.sinks != nullptr && M > -INFINITY) L = L + sink_term(a, head, M);
-    const float inv = L > 0.f ? 1.0f / L : 0.f;
+    const float inv = (L > 0.f ? 1.0f / L : 0.f) * out_gate(a, tok, head);
     elem_t* orow = a.out + ((int64_t)tok * a.nq + head) * a.d;
 #pragma unroll
     for (int dt = 0; dt < NDT; ++dt) {
@@ -1137,8 +1204,8 @@ __global__ __launch_bounds__(256) void attn_prefill_ext_kernel(AttnArgs a, int h
   }
 }
 
-// Decoded tokens: attn_decode_plain_kernel with the four things above; attn_combine_kernel folds its segments.
-template <int DPAD, bool V_LATE>
+// Decoded tokens: attn_decode_plain_kernel with the things above; attn_combine_kernel folds its segments.
+template <int DPAD, bool V_LATE, bool REL>
 __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_decode_ext_kernel(AttnArgs a) {
   constexpr int NDT = DPAD / 16, NQS = DPAD / VK_SLAB;
   const int lane = threadIdx.x & 63;
@@ -1167,6 +1234,7 @@ __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_decode_ext_kernel(AttnA
   c.wave_lo = lo;
   c.keep = keep;
   const int head = kvh * G + ht * 16 + c.r16;
+  init_rel<REL>(c, a, c.row_ok ? head : kvh * G, pos, pos);
   frag_t qf[NQS];
   load_q<NQS>(a, tok, head, c.row_ok, c.g, qf);
   float M = -INFINITY, L = 0.f;
@@ -1174,7 +1242,7 @@ __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_decode_ext_kernel(AttnA
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt) ACC[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int t = t0; t <= t1; ++t)
-    if (t < keep_tiles || t >= tile_lo) tile_step_ext<NDT, NQS, V_LATE>(c, a.scale, a.softcap, qf, t * TILE_KEYS, M, L, ACC);
+    if (t < keep_tiles || t >= tile_lo) tile_step_ext<NDT, NQS, V_LATE, REL>(c, a.scale, a.softcap, qf, t * TILE_KEYS, M, L, ACC);
   if (!c.row_ok) return;
   const int64_t prow = ((int64_t)blockIdx.x * a.nq + head) * a.nseg + seg;
   if (c.g == 0) {
@@ -1191,7 +1259,7 @@ __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_decode_ext_kernel(AttnA
 // Decoded tokens of the same variant where a wave's registers hold two tiles' fragments: attn_decode_seg_kernel's walk
 // (the next tile's keys asked for when this tile's scores are done, its values when this tile's product is), over the
 // tiles of the segment that hold kept first keys or keys of the window.
-template <int DPAD, bool EXACT>
+template <int DPAD, bool EXACT, bool REL>
 __global__ __launch_bounds__(64 * SEG_WAVES, 2) void attn_decode_seg_ext_kernel(AttnArgs a) {
   constexpr int NDT = DPAD / 16, NQS = DPAD / VK_SLAB;
   const int lane = threadIdx.x & 63;
@@ -1227,6 +1295,7 @@ __global__ __launch_bounds__(64 * SEG_WAVES, 2) void attn_decode_seg_ext_kernel(
   c.wave_lo = lo;
   c.keep = keep;
   const int head = kvh * G + ht * 16 + c.r16;
+  init_rel<REL>(c, a, c.row_ok ? head : kvh * G, pos, pos);
   frag_t qf[NQS];
   load_q<NQS>(a, tok, head, c.row_ok, c.g, qf);
   frag_t kf[KSUB][NQS];
@@ -1250,7 +1319,7 @@ __global__ __launch_bounds__(64 * SEG_WAVES, 2) void attn_decode_seg_ext_kernel(
       __builtin_amdgcn_sched_barrier(0);
       if (more) load_keys<NQS, EXACT>(c, next, kf);
       __builtin_amdgcn_sched_barrier(0);
-      tile_softmax_pv_ext<NDT>(c, a.scale, a.softcap, sc, kb, vf, M, L, ACC);
+      tile_softmax_pv_ext<NDT, REL>(c, a.scale, a.softcap, sc, kb, vf, M, L, ACC);
       __builtin_amdgcn_sched_barrier(0);
       if (more) load_values<NDT, EXACT>(c, next, vf);
       __builtin_amdgcn_sched_barrier(0);
@@ -1276,7 +1345,7 @@ __global__ __launch_bounds__(64 * SEG_WAVES, 2) void attn_decode_seg_ext_kernel(
 // weights, which pass through LDS too; then every wave adds up a quarter of the output columns over the four tiles, in
 // order.  Keys and values are all asked for at once, at the start.  The operations on a row's sums, and their order, are those
 // of the kernels above.
-template <int DPAD, bool EXACT>
+template <int DPAD, bool EXACT, bool REL>
 __global__ __launch_bounds__(64 * SEG_TILES, 1) void attn_decode_quad_ext_kernel(AttnArgs a) {
   constexpr int NDT = DPAD / 16, NQS = DPAD / VK_SLAB, ND = NDT / SEG_TILES;   // ND: column blocks of a wave
   __shared__ frag_t probs[SEG_TILES][P_PARTS][KEY_SLABS][64];
@@ -1313,6 +1382,7 @@ __global__ __launch_bounds__(64 * SEG_TILES, 1) void attn_decode_quad_ext_kernel
   c.wave_lo = lo;
   c.keep = keep;
   const int head = kvh * G + ht * 16 + c.r16;
+  init_rel<REL>(c, a, c.row_ok ? head : kvh * G, pos, pos);
   const int first_tile = seg * SEG_TILES;
   const bool mine = (wanted >> wave) & 1u;
   frag_t qf[NQS];
@@ -1337,11 +1407,12 @@ __global__ __launch_bounds__(64 * SEG_TILES, 1) void attn_decode_quad_ext_kernel
   const int kb = (first_tile + wave) * TILE_KEYS;
   float tmax = -INFINITY;
   if (mine) {
+    float rb[REL ? S_PER_LANE : 1];
+    tile_bias<REL>(c, kb, rb);
     tile_scores<NQS, EXACT>(c, kf, qf, sc);
-    const float inner = a.softcap > 0.f ? a.scale / a.softcap : a.scale;
+    natural_scores<REL>(sc, a.scale, a.softcap, rb);
 #pragma unroll
     for (int i = 0; i < S_PER_LANE; ++i) {
-      sc[i] = a.softcap > 0.f ? a.softcap * fast_tanh(sc[i] * inner) : sc[i] * inner;
       const int key = kb + (i / VK_VEC) * VK_SLAB + c.g * VK_VEC + (i % VK_VEC);
       vis[i] = c.row_ok && key <= pos && (key >= lo || key < keep);
       tmax = fmaxf(tmax, vis[i] ? sc[i] : -INFINITY);
@@ -1478,7 +1549,7 @@ __global__ __launch_bounds__(64) void attn_combine_kernel(AttnArgs a) {
     }
   }
   if (a.sinks != nullptr && M > -INFINITY) L = L + sink_term(a, head, M);
-  const float inv = L > 0.f ? 1.0f / L : 0.f;
+  const float inv = (L > 0.f ? 1.0f / L : 0.f) * out_gate(a, tok, head);
   elem_t* orow = a.out + ((int64_t)tok * a.nq + head) * d;
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
@@ -1679,7 +1750,8 @@ int vk_paged_attention(elem_t* out, const elem_t* q, const elem_t* kc, const ele
 static int attention_capped_launch(elem_t* out, const elem_t* q, const elem_t* kc, const elem_t* vc, const int32_t* block_table,
                                    int bt_stride, const int32_t* cu_q, const int32_t* k_len, const int32_t* items, int n_items, int mode,
                                    int nseg, float* scratch, int total_tokens, int nq, int nkv, int d, int P, int window, int keep, int block,
-                                   float scale, float softcap, const void* sinks, int sinks_f32, hipStream_t st) {
+                                   float scale, float softcap, const void* sinks, int sinks_f32, hipStream_t st, const float* rel = nullptr,
+                                   int rel_stride = 0, int rel_far = 0, const elem_t* gate = nullptr, int64_t gate_stride = 0) {
   (void)total_tokens;
   VK_REQUIRE(block >= 0 && (block == 0 || window == 0), "attention: blocks of positions (%d) and a window (%d) exclude each other", block, window);
   VK_REQUIRE(nq > 0 && nkv > 0 && nq % nkv == 0, "attention: %d q heads are not a multiple of %d kv heads", nq, nkv);
@@ -1689,6 +1761,9 @@ static int attention_capped_launch(elem_t* out, const elem_t* q, const elem_t* k
   VK_REQUIRE(keep == 0 || window > 0, "attention: kept first keys need a window");
   VK_REQUIRE(scale > 0.f && softcap >= 0.f, "attention: the score scale must be positive and the cap not negative");
   VK_REQUIRE(mode == 0 || mode == 1, "attention: unknown mode %d", mode);
+  VK_REQUIRE(rel == nullptr || (softcap == 0.f && rel_far >= 0 && rel_stride > rel_far + 2 * REL_PAD && (int64_t)nq * rel_stride < (1ll << 30)),
+             "attention: a bias by distance excludes a cap, and its rows hold %d entries more than its distances", 2 * REL_PAD);
+  VK_REQUIRE(gate == nullptr || gate_stride >= nq, "attention: a gate a head needs rows of at least %d", nq);
   if (n_items <= 0) return 0;
   AttnArgs a;
   a.q = q; a.out = out; a.kc = kc; a.vc = vc; a.block_table = block_table; a.cu_q = cu_q; a.k_len = k_len;
@@ -1696,27 +1771,30 @@ static int attention_capped_launch(elem_t* out, const elem_t* q, const elem_t* k
   a.nseg = nseg; a.scale_log2 = scale * LOG2E;
   a.part_ml = nullptr; a.part_acc = nullptr;
   a.keep = keep; a.scale = scale; a.softcap = softcap; a.sinks = sinks; a.sinks_f32 = sinks_f32; a.block = block;
+  a.rel = rel; a.rel_stride = rel_stride; a.rel_far = rel_far; a.rel_zero = rel_far + REL_PAD; a.gate = gate; a.gate_stride = gate_stride;
   const int G = nq / nkv;
   if (mode == 0 && vk_attn_prefill_shares_tiles(d, P)) {
     // Key and value tiles through LDS, as for the plain attention; eight waves a workgroup unless they are few.
     VK_REQUIRE((int64_t)n_items * (ITEM_ROWS / 16) * nq < (1ll << 31), "attention: too many prompt items");
     const size_t smem = (size_t)4 * TILE_KEYS * d * sizeof(elem_t);
-#define PREFILL_LDS_EXT(DP, NW)                                                                      \
+#define PREFILL_LDS_EXT_OF(DP, NW, REL)                                                              \
   do {                                                                                               \
     static bool raised = false;                                                                      \
     if (!raised) {                                                                                   \
-      (void)hipFuncSetAttribute((const void*)attn_prefill_lds_kernel<DP, NW, 2, true>,               \
+      (void)hipFuncSetAttribute((const void*)attn_prefill_lds_kernel<DP, NW, 2, true, REL>,          \
                                 hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);             \
       raised = true;                                                                                 \
     }                                                                                                \
-    attn_prefill_lds_kernel<DP, NW, 2, true><<<n_items * (ITEM_ROWS / (16 * NW)) * nq, 64 * NW, smem, st>>>(a, n_items); \
+    attn_prefill_lds_kernel<DP, NW, 2, true, REL><<<n_items * (ITEM_ROWS / (16 * NW)) * nq, 64 * NW, smem, st>>>(a, n_items); \
   } while (0)
+#define PREFILL_LDS_EXT(DP, NW) do { if (rel != nullptr) PREFILL_LDS_EXT_OF(DP, NW, true); else PREFILL_LDS_EXT_OF(DP, NW, false); } while (0)
     // (In 32-bit with the widest heads eight waves' registers do not hold the three-part products' operands.)
     const bool four = 2 * (int64_t)n_items * nq < 3 * (int64_t)attn_device_cus() || (sizeof(elem_t) == 4 && d == 256);
     if (d == 64) { if (four) PREFILL_LDS_EXT(64, 4); else PREFILL_LDS_EXT(64, 8); }
     else if (d == 128) { if (four) PREFILL_LDS_EXT(128, 4); else PREFILL_LDS_EXT(128, 8); }
     else { if (four) PREFILL_LDS_EXT(256, 4); else PREFILL_LDS_EXT(256, 8); }
 #undef PREFILL_LDS_EXT
+#undef PREFILL_LDS_EXT_OF
     return vk_check_launch("attention (prompt rows, capped scores, shared tiles)");
   }
   if (mode == 0) {
@@ -1724,9 +1802,15 @@ static int attention_capped_launch(elem_t* out, const elem_t* q, const elem_t* k
     VK_REQUIRE((int64_t)n_items * (ITEM_ROWS / 16) < (1ll << 31), "attention: too many prompt items");
     const dim3 grid(n_items * (ITEM_ROWS / 16), nkv * ((G + hpw - 1) / hpw));
     VK_REQUIRE(grid.y <= 65535, "attention: too many heads");
-    if (d <= 64) attn_prefill_ext_kernel<64><<<grid, 64 * hpw, 0, st>>>(a, hpw);
-    else if (d <= 128) attn_prefill_ext_kernel<128><<<grid, 64 * hpw, 0, st>>>(a, hpw);
-    else attn_prefill_ext_kernel<256><<<grid, 64 * hpw, 0, st>>>(a, hpw);
+#define PREFILL_EXT(DP)                                                                       \
+  do {                                                                                        \
+    if (rel != nullptr) attn_prefill_ext_kernel<DP, true><<<grid, 64 * hpw, 0, st>>>(a, hpw); \
+    else attn_prefill_ext_kernel<DP, false><<<grid, 64 * hpw, 0, st>>>(a, hpw);               \
+  } while (0)
+    if (d <= 64) PREFILL_EXT(64);
+    else if (d <= 128) PREFILL_EXT(128);
+    else PREFILL_EXT(256);
+#undef PREFILL_EXT
     return vk_check_launch("attention (prompt rows, capped scores)");
   }
   VK_REQUIRE(nseg > 0 && nseg <= 65535 && scratch != nullptr, "attention: decode needs nseg in 1..65535 and scratch");
@@ -1737,15 +1821,20 @@ static int attention_capped_launch(elem_t* out, const elem_t* q, const elem_t* k
     // A wave's registers hold two tiles' fragments: the walk with the next tile in flight.
     const bool exact = P >= TILE_KEYS && d == vk_dpad(d);
     const dim3 sgrid(n_items, nkv * ((G + 15) / 16), (nseg + SEG_WAVES - 1) / SEG_WAVES);
-#define DECODE_SEG_EXT(DP)                                                                     \
-  do {                                                                                         \
-    if (exact) attn_decode_seg_ext_kernel<DP, true><<<sgrid, 64 * SEG_WAVES, 0, st>>>(a);      \
-    else attn_decode_seg_ext_kernel<DP, false><<<sgrid, 64 * SEG_WAVES, 0, st>>>(a);           \
+#define DECODE_SEG_EXT_OF(DP, REL)                                                                \
+  do {                                                                                            \
+    if (exact) attn_decode_seg_ext_kernel<DP, true, REL><<<sgrid, 64 * SEG_WAVES, 0, st>>>(a);    \
+    else attn_decode_seg_ext_kernel<DP, false, REL><<<sgrid, 64 * SEG_WAVES, 0, st>>>(a);         \
   } while (0)
+#define DECODE_SEG_EXT(DP) do { if (rel != nullptr) DECODE_SEG_EXT_OF(DP, true); else DECODE_SEG_EXT_OF(DP, false); } while (0)
+#ifdef VK_BF16
     if (d <= 64) DECODE_SEG_EXT(64);
-    else if (d <= 128) DECODE_SEG_EXT(128);
-    else DECODE_SEG_EXT(256);
+    else DECODE_SEG_EXT(128);
+#else
+    DECODE_SEG_EXT(64);
+#endif
 #undef DECODE_SEG_EXT
+#undef DECODE_SEG_EXT_OF
     if (vk_check_launch("attention (decoded rows, capped scores, wave per segment)")) return 1;
     attn_combine_kernel<<<dim3(n_items, nq), 64, 0, st>>>(a);
     return vk_check_launch("attention (combine)");
@@ -1753,23 +1842,31 @@ static int attention_capped_launch(elem_t* out, const elem_t* q, const elem_t* k
 #ifdef VK_BF16
   // (128 < d: the smaller sizes went the way above.)
   const dim3 qgrid(n_items, nkv * ((G + 15) / 16), nseg);
-  if (P >= TILE_KEYS && d == 256) attn_decode_quad_ext_kernel<256, true><<<qgrid, 64 * SEG_TILES, 0, st>>>(a);
-  else attn_decode_quad_ext_kernel<256, false><<<qgrid, 64 * SEG_TILES, 0, st>>>(a);
+  const bool exact = P >= TILE_KEYS && d == 256;
+  if (rel != nullptr) {
+    if (exact) attn_decode_quad_ext_kernel<256, true, true><<<qgrid, 64 * SEG_TILES, 0, st>>>(a);
+    else attn_decode_quad_ext_kernel<256, false, true><<<qgrid, 64 * SEG_TILES, 0, st>>>(a);
+  } else {
+    if (exact) attn_decode_quad_ext_kernel<256, true, false><<<qgrid, 64 * SEG_TILES, 0, st>>>(a);
+    else attn_decode_quad_ext_kernel<256, false, false><<<qgrid, 64 * SEG_TILES, 0, st>>>(a);
+  }
   if (vk_check_launch("attention (decoded rows, capped scores, four waves a segment)")) return 1;
   attn_combine_kernel<<<dim3(n_items, nq), 64, 0, st>>>(a);
   return vk_check_launch("attention (combine)");
 #else
   const dim3 grid(n_items, nkv * ((G + 15) / 16), (nseg + PLAIN_WAVES - 1) / PLAIN_WAVES);
   const bool late = (int64_t)grid.x * grid.y * nseg > 1024;
-#define DECODE_EXT(DP)                                                                   \
-  do {                                                                                   \
-    if (late) attn_decode_ext_kernel<DP, true><<<grid, 64 * PLAIN_WAVES, 0, st>>>(a);    \
-    else attn_decode_ext_kernel<DP, false><<<grid, 64 * PLAIN_WAVES, 0, st>>>(a);        \
+#define DECODE_EXT_OF(DP, REL)                                                                \
+  do {                                                                                        \
+    if (late) attn_decode_ext_kernel<DP, true, REL><<<grid, 64 * PLAIN_WAVES, 0, st>>>(a);    \
+    else attn_decode_ext_kernel<DP, false, REL><<<grid, 64 * PLAIN_WAVES, 0, st>>>(a);        \
   } while (0)
-  if (d <= 64) DECODE_EXT(64);
-  else if (d <= 128) DECODE_EXT(128);
+#define DECODE_EXT(DP) do { if (rel != nullptr) DECODE_EXT_OF(DP, true); else DECODE_EXT_OF(DP, false); } while (0)
+  // (d <= 64 went the way above.)
+  if (d <= 128) DECODE_EXT(128);
   else DECODE_EXT(256);
 #undef DECODE_EXT
+#undef DECODE_EXT_OF
   if (vk_check_launch("attention (decoded rows, capped scores)")) return 1;
   attn_combine_kernel<<<dim3(n_items, nq), 64, 0, st>>>(a);
   return vk_check_launch("attention (combine)");
@@ -1783,6 +1880,20 @@ int vk_paged_attention_capped(elem_t* out, const elem_t* q, const elem_t* kc, co
   return attention_capped_launch(out, q, kc, vc, block_table, bt_stride, cu_q, k_len, items, n_items, mode, nseg, scratch, total_tokens, nq, nkv,
                                  d, P, window, keep, 0, scale, softcap, sinks, sinks_f32, st);
 }
+
+// The same with a bias by distance on the scores (rel [nq, rel_stride] floats or null; a row holds, from its start, REL_PAD
+// entries of the distance rel_far, the distances rel_far .. 0, and REL_PAD entries of the distance 0) and a gate a head (gate
+// [T, gate_stride] elements or null).  vk_attn_rel_pad() is REL_PAD.
+int vk_paged_attention_biased(elem_t* out, const elem_t* q, const elem_t* kc, const elem_t* vc, const int32_t* block_table,
+                              int bt_stride, const int32_t* cu_q, const int32_t* k_len, const int32_t* items, int n_items, int mode,
+                              int nseg, float* scratch, int total_tokens, int nq, int nkv, int d, int P, int window, int keep,
+                              float scale, const void* sinks, int sinks_f32, const float* rel, int rel_stride, int rel_far, const elem_t* gate,
+                              int64_t gate_stride, hipStream_t st) {
+  return attention_capped_launch(out, q, kc, vc, block_table, bt_stride, cu_q, k_len, items, n_items, mode, nseg, scratch, total_tokens, nq, nkv,
+                                 d, P, window, keep, 0, scale, 0.f, sinks, sinks_f32, st, rel, rel_stride, rel_far, gate, gate_stride);
+}
+
+int vk_attn_rel_pad(void) { return REL_PAD; }
 
 // The same kernels with positions cut into blocks of `block`: the row at position p sees key j <= p only if
 // j / block == p / block (integer division), counted from the sequence's first position.  The arithmetic and the

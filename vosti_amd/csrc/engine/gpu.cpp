@@ -159,9 +159,20 @@ struct Kernels::Fn {
   int (*embed_normed)(P, CP, CP, CP, int, int, int, int, float, hipStream_t);
   int (*attention_wide)(P, CP, CP, CP, CP, int, CP, CP, CP, int, int, int, int, int, int, int, float, CP, int, hipStream_t);
   int (*attention_wide_limit)();
+  int (*gemm_act)(P, CP, CP, int, int, int, int64_t, int64_t, int, hipStream_t);
+  int (*gemm_split_act)(P, CP, CP, int, int, int, int64_t, int64_t, int, P, int64_t, hipStream_t);
+  int (*gemm_grouped_act)(P, CP, CP, int, int, int, int64_t, int64_t, CP, int64_t, int, hipStream_t);
+  int (*moe_route_corrected)(P, P, P, CP, CP, CP, int, int, int, int, int, int, int, int, float, hipStream_t);
+  int (*stream_add_norm)(P, P, CP, int, CP, int, int, int, float, hipStream_t);
+  int (*embed_bigram)(P, CP, CP, CP, CP, int, int, int, int64_t, int64_t, int64_t, hipStream_t);
+  int (*qkv_prepare)(CP, int64_t, P, P, P, int, CP, CP, int, int, int, float, CP, int, CP, CP, CP, int64_t, int, int, CP, int, int, int, int, int, int,
+                     hipStream_t);
+  int (*paged_attention_biased)(P, CP, CP, CP, CP, int, CP, CP, CP, int, int, int, P, int, int, int, int, int, int, int, float, CP, int, CP, int, int,
+                                CP, int64_t, hipStream_t);
+  int (*attn_rel_pad)();
 };
 
-static constexpr int KERNEL_ABI = 19;
+static constexpr int KERNEL_ABI = 20;
 
 Kernels::Kernels(const std::string& lib_dir, const std::string& name) : name_(name), fn_(new Fn) {
   if (name == "bf16") dtype_ = DType::BF16;
@@ -206,6 +217,9 @@ Kernels::Kernels(const std::string& lib_dir, const std::string& name) : name_(na
   VK(gated_row_norm, "vk_gated_row_norm"); VK(silu_columns, "vk_silu_columns");
   VK(hyper_in_place, "vk_hyper_in_place"); VK(hyper_step, "vk_hyper_step"); VK(hyper_close, "vk_hyper_close"); VK(embed_normed, "vk_embed_normed");
   VK(attention_wide, "vk_attention_wide"); VK(attention_wide_limit, "vk_attention_wide_limit");
+  VK(gemm_act, "vk_gemm_act"); VK(gemm_split_act, "vk_gemm_split_act"); VK(gemm_grouped_act, "vk_gemm_grouped_act");
+  VK(moe_route_corrected, "vk_moe_route_corrected"); VK(stream_add_norm, "vk_stream_add_norm"); VK(embed_bigram, "vk_embed_bigram");
+  VK(qkv_prepare, "vk_qkv_prepare"); VK(paged_attention_biased, "vk_paged_attention_biased"); VK(attn_rel_pad, "vk_attn_rel_pad");
 #undef VK
   segment_keys_ = fn_->attn_segment_keys();
   item_rows_ = fn_->attn_item_rows();
@@ -366,13 +380,21 @@ void Kernels::fill_random(Tensor& out, uint64_t seed, int kind, float p0, float 
   call(fn_->fill_random(out.data, out.numel(), seed, kind, p0, p1, stream));
 }
 
-Tensor Kernels::gemm(const Tensor& act, const Tensor& w, const Tensor* workspace) {
+Tensor Kernels::gemm(const Tensor& act, const Tensor& w, const Tensor* workspace, int activation) {
   expect(act, "activation", dtype_);
   expect(w, "weight", dtype_);
   if (act.shape.size() != 2 || w.shape.size() != 2 || act.dim(1) != w.dim(1))
     throw EngineError("gemm: activation " + act.describe() + " does not fit weight " + w.describe());
   const int64_t M = act.dim(0), K = act.dim(1), N = w.dim(0);
   Tensor out = empty({M, N});
+  if (activation) {
+    const int64_t need = workspace ? gemm_workspace_floats(M, N, K) : 0;
+    if (need && workspace->dtype == DType::F32 && workspace->numel() >= need)
+      call(fn_->gemm_split_act(out.data, act.data, w.data, (int)M, (int)N, (int)K, K, N, activation, workspace->data, workspace->numel(), stream));
+    else
+      call(fn_->gemm_act(out.data, act.data, w.data, (int)M, (int)N, (int)K, K, N, activation, stream));
+    return out;
+  }
   if (split(out, act, w, false, workspace)) return out;
   call(fn_->gemm(out.data, act.data, w.data, (int)M, (int)N, (int)K, K, N, 0, stream));
   return out;
@@ -894,8 +916,7 @@ Kernels::MoePlan Kernels::moe_route(const Tensor& h, const Tensor& router, int t
   return moe_route_scored(h, router, top, weight_eps, tile_rows, bias, 0);
 }
 
-Kernels::MoePlan Kernels::moe_route_scored(const Tensor& h, const Tensor& router, int top, float weight_eps, int tile_rows, const Tensor* bias,
-                                           int score_kind, int groups, int keep, float scale) {
+Kernels::MoePlan Kernels::empty_plan(const Tensor& h, const Tensor& router, int top, int tile_rows) {
   expect(h, "router input", dtype_);
   expect(router, "router weight", dtype_);
   if (h.shape.size() != 2 || router.shape.size() != 2 || router.dim(1) != h.dim(1) || top < 1 || top > router.dim(0))
@@ -914,6 +935,30 @@ Kernels::MoePlan Kernels::moe_route_scored(const Tensor& h, const Tensor& router
   p.pair_row = empty({T * top}, DType::I32);
   p.tile_expert = empty({tiles}, DType::I32);
   p.expert_start = empty({E + 1}, DType::I32);
+  return p;
+}
+
+void Kernels::fill_plan(MoePlan& p) {
+  call(fn_->moe_plan(p.idx.data, p.row_pair.data, p.row_token.data, p.pair_row.data, p.tile_expert.data, p.expert_start.data, (int)p.idx.dim(0), p.top,
+                     p.experts, p.tile_rows, stream));
+}
+
+Kernels::MoePlan Kernels::moe_route_corrected(const Tensor& h, const Tensor& router, const Tensor& correction, int top, int tile_rows, int groups, int keep,
+                                              int group_score, float scale) {
+  MoePlan p = empty_plan(h, router, top, tile_rows);
+  const int64_t T = h.dim(0), E = router.dim(0);
+  const int cf = norm_weight(correction, "router correction", E);
+  Tensor logits = empty({T, E}, DType::F32);
+  call(fn_->moe_route_corrected(p.idx.data, p.wts.data, logits.data, h.data, router.data, correction.data, cf, (int)T, (int)h.dim(1), (int)E, top, groups,
+                                keep, group_score, scale, stream));
+  fill_plan(p);
+  return p;
+}
+
+Kernels::MoePlan Kernels::moe_route_scored(const Tensor& h, const Tensor& router, int top, float weight_eps, int tile_rows, const Tensor* bias,
+                                           int score_kind, int groups, int keep, float scale) {
+  MoePlan p = empty_plan(h, router, top, tile_rows);
+  const int64_t T = h.dim(0), E = router.dim(0);
   Tensor logits = empty({T, E}, DType::F32);
   if (score_kind != 0 || groups != 1 || scale != 1.f) {
     const int bf = bias ? norm_weight(*bias, "router bias", E) : 0;
@@ -926,8 +971,7 @@ Kernels::MoePlan Kernels::moe_route_scored(const Tensor& h, const Tensor& router
   } else {
     call(fn_->moe_route(p.idx.data, p.wts.data, logits.data, h.data, router.data, (int)T, (int)h.dim(1), (int)E, top, weight_eps, stream));
   }
-  call(fn_->moe_plan(p.idx.data, p.row_pair.data, p.row_token.data, p.pair_row.data, p.tile_expert.data, p.expert_start.data, (int)T, top, (int)E,
-                     tile_rows, stream));
+  fill_plan(p);
   return p;
 }
 
@@ -1102,6 +1146,116 @@ Tensor Kernels::hyper_close(const Tensor& streams, const Tensor* y, const Tensor
   return out;
 }
 
+// ------------------------------------------- a stream's add and norm, pairs of tokens, q k v in other forms
+Tensor Kernels::stream_add_norm(const Tensor& y, Tensor& s, const Tensor& w, float eps) {
+  if (y.dtype != DType::F32) expect(y, "a sublayer's output", dtype_);
+  if (y.shape.size() != 2) throw EngineError("stream add-norm: rows are " + y.describe());
+  expect(s, "stream", DType::F32, y.shape);
+  const int wf = norm_weight(w, "norm weight", y.dim(1));
+  Tensor out = empty(y.shape);
+  call(fn_->stream_add_norm(out.data, s.data, y.data, y.dtype == DType::F32 ? 1 : 0, w.data, wf, (int)y.dim(0), (int)y.dim(1), eps, stream));
+  return out;
+}
+
+Tensor Kernels::embed_bigram(const Tensor& table, const Tensor& pairs, const Tensor& ids, const Tensor& before, int64_t mul_before, int64_t mul_own) {
+  expect(table, "embedding table", dtype_);
+  expect(pairs, "table of pairs", dtype_);
+  if (table.shape.size() != 2 || pairs.shape.size() != 2 || pairs.dim(1) != table.dim(1) || pairs.dim(0) < 2)
+    throw EngineError("bigram embedding: tables " + table.describe() + " and " + pairs.describe());
+  const int64_t V = table.dim(0), H = table.dim(1), T = ids.numel();
+  expect(ids, "ids", DType::I32, {T});
+  expect(before, "ids before", DType::I32, {T});
+  Tensor out = empty({T, H}, DType::F32);
+  call(fn_->embed_bigram(out.data, table.data, pairs.data, ids.data, before.data, (int)T, (int)H, (int)V, mul_before, mul_own, pairs.dim(0) - 1, stream));
+  return out;
+}
+
+Tensor Kernels::qkv_prepare(const Tensor& qkv, int nq, int nkv, int d, int size, int vsize, const Prepare& how, const Tensor& k_cache,
+                            const Tensor& v_cache, int page_size, const Tensor& positions, const Tensor& slots) {
+  expect(qkv, "qkv", dtype_);
+  const int64_t W = (int64_t)(nq + 2 * nkv) * d;
+  if (qkv.shape.size() != 2 || qkv.dim(1) < W) throw EngineError("qkv_prepare: rows are " + qkv.describe() + ", expected a width of at least " + std::to_string(W));
+  const int64_t T = qkv.dim(0);
+  int wf = 0;
+  if (how.norm == 1 || how.norm == 3) {
+    if (!how.q_w || !how.k_w) throw EngineError("qkv_prepare: the norms' weights are missing");
+    wf = norm_weight(*how.q_w, "q norm weight", how.norm == 1 ? size : (int64_t)nq * size);
+    if (norm_weight(*how.k_w, "k norm weight", how.norm == 1 ? size : (int64_t)nkv * size) != wf)
+      throw EngineError("qkv_prepare: q and k norm weights must have the same type");
+  }
+  if (how.inv_freq) {
+    expect(*how.inv_freq, "rotation frequencies", DType::F32);
+    if (how.inv_freq->shape.size() != 1 || how.inv_freq->dim(0) < 1 || 2 * how.inv_freq->dim(0) > size)
+      throw EngineError("qkv_prepare: rotation frequencies are " + how.inv_freq->describe() + " for heads of " + std::to_string(size));
+  }
+  expect(positions, "positions", DType::I32, {T});
+  expect(slots, "slots", DType::I32, {T});
+  if (k_cache.shape.size() != 4) throw EngineError("k cache is " + k_cache.describe());
+  const int64_t pages = k_cache.dim(0);
+  expect(k_cache, "k cache", dtype_, {pages, nkv, page_size, d});
+  expect(v_cache, "v cache", dtype_, {pages, nkv, d, page_size});
+  int sf = 0;
+  const void* v0 = nullptr;
+  if (how.share) {
+    sf = norm_weight(how.share->view({how.share->numel()}), "values' share", 1);
+    expect(how.v0, "the first values' rows", dtype_);
+    if (how.v0.shape.size() != 2 || how.v0.dim(0) != T || how.v0_size < 1 || how.v0_d < how.v0_size || how.v0_col < 0 || (nkv * vsize) % how.v0_size ||
+        how.v0_col + (int64_t)(nkv * vsize / how.v0_size) * how.v0_d > how.v0.dim(1))
+      throw EngineError("qkv_prepare: the first values' rows are " + how.v0.describe());
+    v0 = static_cast<const char*>(how.v0.data) + (size_t)how.v0_col * dtype_bytes(dtype_);
+  }
+  Tensor q = empty({T, nq, d});
+  call(fn_->qkv_prepare(qkv.data, qkv.dim(1), q.data, k_cache.data, v_cache.data, how.norm, how.q_w ? how.q_w->data : nullptr,
+                        how.k_w ? how.k_w->data : nullptr, wf, size, vsize, how.eps, how.inv_freq ? how.inv_freq->data : nullptr,
+                        how.inv_freq ? (int)how.inv_freq->dim(0) : 0, positions.data, slots.data, v0, v0 ? how.v0.dim(1) : 0, how.v0_d, how.v0_size,
+                        v0 ? how.share->data : nullptr, sf, (int)T, nq, nkv, d, page_size, stream));
+  return q;
+}
+
+void Kernels::paged_attention_biased(Tensor& out, const Tensor& q, const Tensor& k_cache, const Tensor& v_cache, const Tensor& block_table,
+                                     const Tensor& cu_q, const Tensor& k_len, const Tensor& items, int mode, float scale, int window, const Tensor* rel,
+                                     int far, const Tensor* gate, int64_t gate_col, int max_k_len, int nseg, const Tensor* scratch) {
+  expect(q, "q", dtype_);
+  expect(block_table, "block table", DType::I32);
+  if (q.shape.size() != 3 || k_cache.shape.size() != 4 || block_table.shape.size() != 2)
+    throw EngineError("attention: q " + q.describe() + ", k cache " + k_cache.describe() + ", block table " + block_table.describe());
+  const int64_t T = q.dim(0), nq = q.dim(1), d = q.dim(2), pages = k_cache.dim(0), nkv = k_cache.dim(1), P = k_cache.dim(2);
+  const int64_t S = block_table.dim(0), W = block_table.dim(1);
+  expect(k_cache, "k cache", dtype_, {pages, nkv, P, d});
+  expect(v_cache, "v cache", dtype_, {pages, nkv, d, P});
+  expect(cu_q, "cu_q", DType::I32, {S + 1});
+  expect(k_len, "k_len", DType::I32, {S});
+  expect(out, "attention output", dtype_, q.shape);
+  if (items.shape.size() != 2 || items.dim(1) != 2) throw EngineError("attention: items are " + items.describe());
+  expect(items, "items", DType::I32);
+  if (mode != 0 && mode != 1) throw EngineError("attention with biased scores: mode " + std::to_string(mode));
+  if (W * P < max_k_len)
+    throw EngineError("attention: a block table of " + std::to_string(W) + " pages of " + std::to_string(P) + " does not cover " +
+                      std::to_string(max_k_len) + " keys");
+  if (rel) expect(*rel, "biases by distance", DType::F32, {nq, (int64_t)far + 1 + 2 * distance_pad()});
+  if (gate) {
+    expect(*gate, "heads' gates", dtype_);
+    if (gate->shape.size() != 2 || gate->dim(0) != T || gate_col < 0 || gate_col + nq > gate->dim(1)) throw EngineError("attention: the heads' gates are " + gate->describe());
+  }
+  void* sp = nullptr;
+  const int64_t n_items = items.dim(0);
+  if (mode == 1) {
+    if (nseg < (max_k_len + segment_keys_ - 1) / segment_keys_)
+      throw EngineError("attention: " + std::to_string(nseg) + " segments do not cover " + std::to_string(max_k_len) + " keys");
+    const int64_t need = attn_scratch_floats((int)n_items, (int)nq, (int)d, nseg);
+    if (!scratch || scratch->dtype != DType::F32 || scratch->numel() < need)
+      throw EngineError("attention: scratch of " + std::to_string(need) + " floats needed");
+    sp = scratch->data;
+  }
+  call(fn_->paged_attention_biased(out.data, q.data, k_cache.data, v_cache.data, block_table.data, (int)W, cu_q.data, k_len.data, items.data,
+                                   (int)n_items, mode, nseg, sp, (int)T, (int)nq, (int)nkv, (int)d, (int)P, window, 0, scale, nullptr, 0,
+                                   rel ? rel->data : nullptr, rel ? (int)rel->dim(1) : 0, far,
+                                   gate ? static_cast<const char*>(gate->data) + (size_t)gate_col * dtype_bytes(dtype_) : nullptr, gate ? gate->dim(1) : 0,
+                                   stream));
+}
+
+int Kernels::distance_pad() const { return fn_->attn_rel_pad(); }
+
 int Kernels::attention_limit() const { return fn_->attention_wide_limit(); }
 
 Tensor Kernels::qkv_post_norm_angles_paired(const Tensor& qkv, int nq, int nkv, int d, const Tensor* k_cache, const Tensor* v_cache, int page_size,
@@ -1207,15 +1361,15 @@ void Kernels::relu_square(Tensor& x) {
 
 bool Kernels::gemm_grouped_takes(int64_t K) const { return K % (dtype_ == DType::BF16 ? 64 : 32) == 0; }
 
-Tensor Kernels::gemm_grouped(const Tensor& act, const Tensor& w, const Tensor& block_weights) {
+Tensor Kernels::gemm_grouped(const Tensor& act, const Tensor& w, const Tensor& block_weights, int activation) {
   expect(act, "activation", dtype_);
   expect(w, "weights", dtype_);
   if (act.shape.size() != 2 || w.shape.size() != 3 || act.dim(1) != w.dim(2) || act.dim(0) % 128 || !gemm_grouped_takes(act.dim(1)))
     throw EngineError("grouped gemm: activation " + act.describe() + ", weights " + w.describe());
   expect(block_weights, "the blocks' matrices", DType::I32, {act.dim(0) / 128});
   Tensor out = empty({act.dim(0), w.dim(1)});
-  call(fn_->gemm_grouped(out.data, act.data, w.data, (int)act.dim(0), (int)w.dim(1), (int)w.dim(2), act.dim(1), w.dim(1), block_weights.data,
-                         w.dim(1) * w.dim(2), stream));
+  call(fn_->gemm_grouped_act(out.data, act.data, w.data, (int)act.dim(0), (int)w.dim(1), (int)w.dim(2), act.dim(1), w.dim(1), block_weights.data,
+                             w.dim(1) * w.dim(2), activation, stream));
   return out;
 }
 

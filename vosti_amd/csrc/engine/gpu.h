@@ -120,8 +120,8 @@ class Kernels {
   // scaled by p0, kind 1: p0 + u * p1.
   void fill_random(Tensor& out, uint64_t seed, int kind, float p0, float p1);
   // act @ w^T, w [out, in].  workspace: float32 scratch; with enough of it (gemm_workspace_floats) some sizes
-  // take a faster route to the same bits.
-  Tensor gemm(const Tensor& act, const Tensor& w, const Tensor* workspace = nullptr);
+  // take a faster route to the same bits.  activation 1: the square of max(., 0) on the rounded outputs, in the same launch.
+  Tensor gemm(const Tensor& act, const Tensor& w, const Tensor* workspace = nullptr, int activation = 0);
   Tensor gemm_swiglu(const Tensor& act, const Tensor& w_gate_up, const Tensor* workspace = nullptr);
   // float32 elements of workspace with which gemm / gemm_swiglu take the route through chunk sums for these
   // sizes, or 0 where that route does not exist or is the slower one.
@@ -229,13 +229,17 @@ class Kernels {
   Tensor moe_sum(const Tensor& y, const MoePlan& plan, const Tensor* extra = nullptr);   // extra [T, width] elements: added last
   // act [M, K] in blocks of 128 rows, block b times the matrix block_weights[b] of w [matrices, N, K] (negative: the
   // block is skipped); [M, N] elements, the bits gemm gives for the same rows and matrix.  K in whole pairs of slabs.
-  Tensor gemm_grouped(const Tensor& act, const Tensor& w, const Tensor& block_weights);
+  Tensor gemm_grouped(const Tensor& act, const Tensor& w, const Tensor& block_weights, int activation = 0);
   bool gemm_grouped_takes(int64_t K) const;
   // moe_route with a choice of score: 0 as moe_route; 1: a chosen expert's weight is the logistic function of its logit.
   // 2: the softmax over all experts as it is.  groups, keep: only experts of the `keep` best of that many equal groups can be
   // chosen; scale: on every weight.
   MoePlan moe_route_scored(const Tensor& h, const Tensor& router, int top, float weight_eps, int tile_rows, const Tensor* bias, int score_kind,
                            int groups = 1, int keep = 1, float scale = 1.f);
+  // moe_route_scored with score 1 and a correction [experts] that joins the scores for the choice alone; group_score 0: a group is
+  // worth its largest corrected score, 1: the sum of its two largest.
+  MoePlan moe_route_corrected(const Tensor& h, const Tensor& router, const Tensor& correction, int top, int tile_rows, int groups, int keep,
+                              int group_score, float scale);
   // moe_glu for experts that read their input times the pair's weight: every row's gate and up values are multiplied by
   // its pair's weight before the clamps; moe_sum_unweighed then adds a token's rows as they are.
   Tensor moe_glu_weighed(const Tensor& gate_up, float limit, float slope, float shift, const MoePlan& plan);
@@ -276,6 +280,31 @@ class Kernels {
   Tensor hyper_step(Tensor& streams, const Tensor* y, const Tensor* back, const Tensor& take, int S, const Tensor* w, float eps);
   // The sum of the streams of the rows that are asked for, after the last output: floats [rows, W].
   Tensor hyper_close(const Tensor& streams, const Tensor* y, const Tensor* back, int S, const Tensor& rows);
+  // ---- a stream that takes in a sublayer's output where the next one reads it; an embedding of pairs of tokens (stream.hip)
+  // stream <- stream + y (elements or floats), in place; returns norm(stream) * w as elements.
+  Tensor stream_add_norm(const Tensor& y, Tensor& stream, const Tensor& w, float eps);
+  // table[ids] + pairs[(before * mul_before + ids * mul_own) mod buckets] as floats [T, width]; the last row of pairs where before < 0.
+  Tensor embed_bigram(const Tensor& table, const Tensor& pairs, const Tensor& ids, const Tensor& before, int64_t mul_before, int64_t mul_own);
+  // ---- from the projections to attention in one launch, in the forms that qkv_post has not (qkv_prepare.hip)
+  struct Prepare {
+    int norm = 0;                                // 0: none; 1: a head, weighted; 2: a head, after the rotation, no weight; 3: all heads together, weighted
+    const Tensor *q_w = nullptr, *k_w = nullptr;
+    float eps = 0.f;
+    const Tensor* inv_freq = nullptr;            // null: no rotation
+    const Tensor* share = nullptr;               // [1]: v <- (1 - share) v + share v0; null: v stays
+    Tensor v0;                                   // the rows that hold v0 ...
+    int64_t v0_col = 0;                          // ... from this column on, in heads of v0_d columns of which v0_size count
+    int v0_d = 0, v0_size = 0;
+  };
+  // qkv [T, >= (nq + 2 nkv) d]; size, vsize: the heads' own entries.  Stores k and v, returns q [T, nq, d].
+  Tensor qkv_prepare(const Tensor& qkv, int nq, int nkv, int d, int size, int vsize, const Prepare& how, const Tensor& k_cache, const Tensor& v_cache,
+                     int page_size, const Tensor& positions, const Tensor& slots);
+  // paged_attention_capped without a cap: a bias by distance on the scores (rel [nq, far + 1 + 2 pad] floats as the kernels read them,
+  // or null) and a gate a head (the columns [gate_col, gate_col + nq) of gate, or null).
+  void paged_attention_biased(Tensor& out, const Tensor& q, const Tensor& k_cache, const Tensor& v_cache, const Tensor& block_table,
+                              const Tensor& cu_q, const Tensor& k_len, const Tensor& items, int mode, float scale, int window, const Tensor* rel,
+                              int far, const Tensor* gate, int64_t gate_col, int max_k_len, int nseg, const Tensor* scratch);
+  int distance_pad() const;                      // entries a row of rel holds beyond its distances, at either end
   // The widest cached row that attention takes; rows of more than 256 entries go through vector arithmetic.
   int attention_limit() const;
   void relu_square(Tensor& x);                 // x <- max(x, 0)^2
@@ -286,6 +315,8 @@ class Kernels {
   void call(int rc) const;
   void expect(const Tensor& t, const char* what, DType dtype, std::vector<int64_t> shape = {}) const;
   int norm_weight(const Tensor& w, const char* what, int64_t n) const;   // 1 if the weight is float32
+  MoePlan empty_plan(const Tensor& h, const Tensor& router, int top, int tile_rows);   // a plan's arrays, not yet written
+  void fill_plan(MoePlan& p);                                                          // from the choices to the rows' places
   bool split(Tensor& out, const Tensor& act, const Tensor& w, bool swiglu, const Tensor* workspace);
 
   std::string name_;

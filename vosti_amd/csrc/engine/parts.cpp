@@ -215,6 +215,14 @@ std::vector<float> host_floats(const Tensor& w) {
   return out;
 }
 
+// Floats, times a factor, on the GPU.
+Tensor float_tensor(std::vector<float> v, float factor = 1.f) {
+  for (float& x : v) x *= factor;
+  Tensor out = zero_weight({(int64_t)v.size()}, DType::F32);
+  if (!v.empty()) hip_check(hipMemcpy(out.data, v.data(), v.size() * sizeof(float), hipMemcpyHostToDevice), "writing a weight");
+  return out;
+}
+
 int64_t round_up(int64_t n, int64_t to) { return (n + to - 1) / to * to; }
 
 // h[t] = E[ids[t]], a row copy without scale (src/exec/dense_swiglu_model.rs:271-273).
@@ -292,17 +300,58 @@ class NormedEmbedding : public Embedding {
   Tensor weight_, norm_;
 };
 
+// h[t] = E[ids[t]] + P[row of (the token before, ids[t])], as the residual stream in 32-bit: a second table whose row a hash of a
+// token and its predecessor picks, (before * mul_prev + own * mul_cur) mod buckets; a request's first token takes row
+// `buckets`, the last.
+class BigramEmbedding : public Embedding {
+ public:
+  BigramEmbedding(const PartSpec& s, Kernels& k)
+      : Embedding(k), vocab_(s.integer("vocab_size")), hidden_(s.integer("hidden_size")), buckets_(s.integer("buckets")), mul_prev_(s.integer("mul_prev")),
+        mul_cur_(s.integer("mul_cur")) {
+    if (buckets_ < 1) throw ConfigError("an embedding of pairs needs at least one bucket");
+  }
+  std::vector<ParamDecl> params() const override { return {{"weight", {vocab_, hidden_}}, {"bigram", {buckets_ + 1, hidden_}}}; }
+  void load(std::map<std::string, Tensor>& t) override {
+    weight_ = need(t, "weight");
+    bigram_ = need(t, "bigram");
+  }
+  const char* step_inputs_key() const override { return "embedding.before"; }
+  void step_inputs(HostStep& step, std::vector<std::pair<std::string, HostArray>>& out) override {
+    HostArray a;
+    size_t at = 0;
+    for (size_t s = 0; s < step.q_lens.size(); ++s)
+      for (int i = 0; i < step.q_lens[s]; ++i, ++at) a.data.push_back(i == 0 ? step.before[s] : step.ids[at - 1]);
+    a.shape = {(int64_t)a.data.size()};
+    out.emplace_back("embedding.before", std::move(a));
+  }
+  Tensor forward(const Tensor&) override { throw EngineError("an embedding of pairs needs the tokens before the step's"); }
+  Tensor forward(const Tensor& ids, StepContext& ctx) override {
+    return kernels.embed_bigram(weight_, bigram_, ids, ctx.inputs.at("embedding.before"), mul_prev_, mul_cur_);
+  }
+
+ private:
+  int64_t vocab_, hidden_, buckets_, mul_prev_, mul_cur_;
+  Tensor weight_, bigram_;
+};
+
 // y = (x * rsqrt(mean(x^2) + eps)) * w in 32-bit (kernels/triton_kernels/rmsnorm.py:63-93); with a residual
 // the norm sees the unrounded sum (kernels/triton_kernels/rmsnorm_residual.py:73-125).
 class RMSNorm : public Norm {
  public:
   // offset: the weight that multiplies is offset + w (1 for a weight that is stored around zero, 0 by default).
-  RMSNorm(const PartSpec& s, Kernels& k) : Norm(k), size_(s.integer("size")), eps_((float)s.number("eps")), offset_((float)s.number("offset", 0.0)) {}
+  // scale: on every output (a constant on what is projected from them), as a 32-bit weight times it.
+  RMSNorm(const PartSpec& s, Kernels& k)
+      : Norm(k), size_(s.integer("size")), eps_((float)s.number("eps")), offset_((float)s.number("offset", 0.0)), scale_(s.number("scale", 1.0)) {
+    if (offset_ != 0.f && scale_ != 1.0) throw ConfigError("a norm with a weight offset has no scale");
+  }
   std::vector<ParamDecl> params() const override {
     if (offset_ != 0.f) return {{"weight", {size_}, true, true, -0.1, 0.1}};
     return {{"weight", {size_}, true, true, 0.9, 1.1}};
   }
-  void load(std::map<std::string, Tensor>& t) override { weight_ = need(t, "weight"); }
+  void load(std::map<std::string, Tensor>& t) override {
+    weight_ = need(t, "weight");
+    if (scale_ != 1.0) weight_ = float_tensor(host_floats(weight_), (float)scale_);
+  }
   // Rows of a 32-bit residual stream are read as they are; the result is elements either way.
   Tensor forward(const Tensor& x) override {
     if (offset_ != 0.f || x.dtype != kernels.dtype()) return kernels.stream_norm(x, weight_, eps_, offset_);
@@ -310,6 +359,7 @@ class RMSNorm : public Norm {
   }
   Tensor forward_add(const Tensor& x, Tensor& residual) override {
     if (offset_ != 0.f) throw EngineError("a norm with a weight offset has no fused residual add in the element type");
+    if (residual.dtype == DType::F32 && kernels.dtype() != DType::F32) return kernels.stream_add_norm(x, residual, weight_, eps_);
     return kernels.add_rmsnorm(x, residual, weight_, eps_);
   }
   void forward_scaled_add(const Tensor& y, const Tensor& base, Tensor& out, float mult, Tensor* rounded) override {
@@ -321,6 +371,7 @@ class RMSNorm : public Norm {
  private:
   int64_t size_;
   float eps_, offset_;
+  double scale_;
   Tensor weight_;
 };
 
@@ -381,7 +432,8 @@ class Rotary : public PositionEncoding {
 // The same half-rotation with angles that are computed where they are used, in 32-bit, and frequencies whose long
 // wavelengths are stretched (rotary_stretched_frequencies has the rule): numbers rotary_dim, theta and, for a stretch,
 // factor, original, fast, slow.  Cosine and sine are multiplied by 0.1 ln(factor) + 1.  linear_factor instead of factor:
-// every frequency is divided by it and nothing else changes (rotary_linear_frequencies).  neighbours 1: a pair is a head's
+// every frequency is divided by it and nothing else changes (rotary_linear_frequencies).  band_factor, original, band_low,
+// band_high: the frequencies are divided by bands of their wavelength (rotary_banded_frequencies).  neighbours 1: a pair is a head's
 // elements 2c and 2c + 1 instead of c and c + half.
 class RotaryStretched : public PositionEncoding {
  public:
@@ -392,7 +444,10 @@ class RotaryStretched : public PositionEncoding {
     neighbours_ = s.integer("neighbours", 0) != 0;
     const double linear = s.number("linear_factor", 0.0);
     if (linear < 0 || (linear > 0 && s.number("factor", 0.0) > 0)) throw ConfigError("a rotation is stretched by 'factor' or by 'linear_factor', not both");
-    if (linear > 0) rotary_linear_frequencies(s.number("theta"), (int)rotary_dim_, linear, f.data());
+    const double banded = s.number("band_factor", 0.0);
+    if (banded > 0 && (linear > 0 || s.number("factor", 0.0) > 0)) throw ConfigError("a rotation is stretched in one way");
+    if (banded > 0) rotary_banded_frequencies(s.number("theta"), (int)rotary_dim_, banded, s.number("original"), s.number("band_low"), s.number("band_high"), f.data());
+    else if (linear > 0) rotary_linear_frequencies(s.number("theta"), (int)rotary_dim_, linear, f.data());
     else
       mag_ = rotary_stretched_frequencies(s.number("theta"), (int)rotary_dim_, s.number("factor", 0.0), s.number("original", 1.0), s.number("fast", 1.0),
                                           s.number("slow", 1.0), f.data());
@@ -458,7 +513,12 @@ AttentionItems& attention_items(Kernels& kernels, HostStep& step) {
 // value projections: it always reads another execution's cache), block (positions are cut into blocks of this many from
 // the sequence's start, and a query sees the earlier keys of its own block only; sink 2 is the constant 0 as every
 // head's sink), output_gate (the heads' outputs are multiplied element by element with sigmoid(W_gate h), a projection of
-// the mixer's own input, before the output projection).  The cache and the kernels see one head size: the
+// the mixer's own input, before the output projection), head_gate (a head's output is multiplied by sigmoid(w_gate[head] . h),
+// one number a head), unit_norm with eps (after the rotation every q and k head is divided by its root mean square),
+// whole_norm (q_norm and k_norm are norms over all heads' entries together), distance_bias with bias_max (a learned number per
+// head and class of distances is added to the scaled score; distance_class has the classes, the stored table their number),
+// value_mix (1: this layer's values are what later layers mix with; 2: v <- (1 - share) v + share v_first with a learned share
+// and those values of the same token, before they are cached).  The cache and the kernels see one head size: the
 // larger of the two, rounded up to 16; the shorter of keys and values is padded with zeros in the weights, so that
 // the projections write the padding and the output projection ignores it.
 class Attention : public Mixer {
@@ -468,7 +528,10 @@ class Attention : public Mixer {
         dk_((int)s.integer("head_dim")), dv_((int)s.integer("value_dim", s.integer("head_dim"))), scale_((float)s.number("scale")),
         window_((int)s.integer("window", 0)), keep_((int)s.integer("keep_first", 0)), softcap_((float)s.number("softcap", 0.0)),
         bias_(s.integer("bias", 0) != 0), sink_((int)s.integer("sink", 0)), exact_(s.integer("exact_weights", 0) != 0),
-        own_kv_(s.integer("own_kv", 1) != 0), block_((int)s.integer("block", 0)), gate_(s.integer("output_gate", 0) != 0) {
+        own_kv_(s.integer("own_kv", 1) != 0), block_((int)s.integer("block", 0)), gate_(s.integer("output_gate", 0) != 0),
+        head_gate_(s.integer("head_gate", 0) != 0), unit_(s.integer("unit_norm", 0) != 0), whole_(s.integer("whole_norm", 0) != 0),
+        bias_by_distance_(s.integer("distance_bias", 0) != 0), mix_((int)s.integer("value_mix", 0)), unit_eps_((float)s.number("eps", 0.0)),
+        bias_max_(s.number("bias_max", 0.0)) {
     d_ = (int)round_up(std::max(dk_, dv_), 16);
     if (nq_ % nkv_) throw ConfigError(std::to_string(nq_) + " heads are not a multiple of " + std::to_string(nkv_) + " kv heads");
     if (dk_ < 1 || dv_ < 1 || d_ > 256)
@@ -481,7 +544,19 @@ class Attention : public Mixer {
     if (const PartSpec* p = s.part("position")) position_ = build_part<PositionEncoding>("position", *p, k);
     if (bias_ && (q_norm_ || k_norm_ || position_))
       throw ConfigError("attention: biases are not built together with head norms or a position encoding");
+    if (mix_ < 0 || mix_ > 2) throw ConfigError("attention: 'value_mix' is 0 (none), 1 (the first values) or 2 (a blend with them)");
+    if (prepared() && (bias_ || !own_kv_ || gate_)) throw ConfigError("attention: unit or whole norms and mixed values are built for layers with keys of their own, without biases and output gates an element");
+    if (unit_ && (q_norm_ || k_norm_)) throw ConfigError("attention: unit norms exclude weighted ones");
+    if ((whole_ || padded_norms_alone()) && (!q_norm_ || !k_norm_)) throw ConfigError("attention: norms of q and k come together here");
+    if (whole_ && position_) throw ConfigError("attention: a norm over all heads is built without a rotation");
+    if ((bias_by_distance_ || head_gate_) && (softcap_ > 0.f || keep_ > 0 || sink_ || block_ > 0 || gate_))
+      throw ConfigError("attention: a bias by distance or a gate a head is built without caps, kept keys, sinks, blocks and output gates an element");
   }
+  // Head norms on padded heads without a rotation.
+  bool padded_norms_alone() const { return d_ != dk_ && (q_norm_ || k_norm_) && !position_; }
+  // What stands between the projections and attention is one launch of qkv_prepare.
+  bool prepared() const { return unit_ || whole_ || mix_ || padded_norms_alone(); }
+  bool biased() const { return bias_by_distance_ || head_gate_; }
   // The kernel with capped scores serves every one of these.
   bool capped() const { return softcap_ > 0.f || keep_ > 0 || sink_ || exact_ || block_ > 0; }
   std::vector<ParamDecl> params() const override {
@@ -502,6 +577,17 @@ class Attention : public Mixer {
       p.push_back(sinks);
     }
     if (gate_) p.push_back({"gate_proj.weight", {(int64_t)nq_ * dv_, hidden_}});
+    if (head_gate_) p.push_back({"head_gate.weight", {(int64_t)nq_, hidden_}});
+    if (bias_by_distance_) {
+      ParamDecl rel{"distance_bias", {-1, (int64_t)nq_}};
+      rel.p0 = 1.0;
+      rel.free_size = 32;
+      p.push_back(rel);
+    }
+    if (mix_ == 2) {
+      ParamDecl share{"value_share", {}, true, true, 0.3, 0.7};
+      p.push_back(share);
+    }
     return p;
   }
   std::vector<std::pair<std::string, Part*>> children() override {
@@ -521,7 +607,10 @@ class Attention : public Mixer {
     }
     // The output gate's rows follow the heads', so that the steps between the projections read the heads where they were.
     if (gate_) rows.push_back(pad_row_blocks(need(t, "gate_proj.weight"), nq_, dv_, d_));
+    if (head_gate_) rows.push_back(pad_matrix(need(t, "head_gate.weight"), round_up(nq_, 8), hidden_));
     w_qkv_ = rows.size() > 1 ? stack_rows(rows) : rows[0];
+    if (bias_by_distance_) load_distances(need(t, "distance_bias"));
+    if (mix_ == 2) share_ = need(t, "value_share");
     w_o_ = pad_column_blocks(need(t, "o_proj.weight"), nq_, dv_, d_);
     if (bias_) {
       std::vector<Tensor> b = {pad_row_blocks(need(t, "q_proj.bias"), nq_, dk_, d_)};
@@ -564,7 +653,7 @@ class Attention : public Mixer {
   }
   // Workspace with which the two projections of T rows take their faster route, where there is one.
   int64_t gemm_floats(int64_t T) const {
-    return std::max(kernels.gemm_workspace_floats(T, (int64_t)(nq_ + 2 * nkv_ + (gate_ ? nq_ : 0)) * d_, hidden_),
+    return std::max(kernels.gemm_workspace_floats(T, (int64_t)(nq_ + 2 * nkv_ + (gate_ ? nq_ : 0)) * d_ + (head_gate_ ? round_up(nq_, 8) : 0), hidden_),
                     kernels.gemm_workspace_floats(T, hidden_, (int64_t)nq_ * d_));
   }
   int64_t workspace_floats(HostStep& step) override {
@@ -598,11 +687,13 @@ class Attention : public Mixer {
     else throw EngineError("an attention layer with an output gate and projections of its own cannot read another execution's cache");
     const bool padded_norm = d_ != dk_ && (q_norm_ || k_norm_);
     const bool norm_angles = position_ && position_->angle_frequencies() && (q_norm_ || k_norm_) && fused();
-    if (padded_norm && !norm_angles) throw ConfigError("attention: head norms on padded head sizes are built for rotations by computed angles only");
+    if (padded_norm && !norm_angles && !prepared()) throw ConfigError("attention: head norms on padded head sizes are built for rotations by computed angles only");
     // The kernels between the projections take rows of exactly the heads' width, except the one that says otherwise.
-    const Tensor qkv = (qkv_all.dim(1) == heads_w || norm_angles) ? qkv_all : k.columns(qkv_all, 0, heads_w);
+    const Tensor qkv = (qkv_all.dim(1) == heads_w || norm_angles || prepared()) ? qkv_all : k.columns(qkv_all, 0, heads_w);
     Tensor q;
-    if (norm_angles) {
+    if (prepared()) {
+      q = prepare(qkv, ctx, cache, tables);
+    } else if (norm_angles) {
       const Norm* en = q_norm_ ? q_norm_.get() : k_norm_.get();
       q = k.qkv_post_norm_angles_paired(qkv, nq_, cache.writable ? nkv_ : 0, d_, &cache.k, &cache.v, cache.page_size,
                                         q_norm_ ? q_norm_->row_scale_weight() : nullptr, k_norm_ && cache.writable ? k_norm_->row_scale_weight() : nullptr,
@@ -630,8 +721,12 @@ class Attention : public Mixer {
     const Tensor& prefill_items = ctx.inputs.at("attention.prefill_items");
     const Tensor& decode_items = ctx.inputs.at("attention.decode_items");
     const Tensor* sinks = sink_ ? &sinks_ : nullptr;
+    const Tensor *rel = bias_by_distance_ ? &rel_ : nullptr, *head_gate = head_gate_ ? &qkv_all : nullptr;
     if (prefill_items.dim(0)) {
-      if (capped())
+      if (biased())
+        k.paged_attention_biased(out, q, cache.k, cache.v, tables.block_table, ctx.cu_q, ctx.k_len, prefill_items, 0, scale_, window_, rel, far_,
+                                 head_gate, heads_w, ctx.host->k_len_bound, 0, nullptr);
+      else if (capped())
         k.paged_attention_capped(out, q, cache.k, cache.v, tables.block_table, ctx.cu_q, ctx.k_len, prefill_items, 0, scale_, window_, keep_,
                                  softcap_, sinks, ctx.host->k_len_bound, 0, nullptr, block_);
       else
@@ -640,7 +735,10 @@ class Attention : public Mixer {
     }
     if (decode_items.dim(0)) {
       const Tensor scratch = ctx.workspace(k.attn_scratch_floats((int)decode_items.dim(0), nq_, d_, m.nseg));
-      if (capped())
+      if (biased())
+        k.paged_attention_biased(out, q, cache.k, cache.v, tables.block_table, ctx.cu_q, ctx.k_len, decode_items, 1, scale_, window_, rel, far_,
+                                 head_gate, heads_w, m.decode_bound, m.nseg, &scratch);
+      else if (capped())
         k.paged_attention_capped(out, q, cache.k, cache.v, tables.block_table, ctx.cu_q, ctx.k_len, decode_items, 1, scale_, window_, keep_,
                                  softcap_, sinks, m.decode_bound, m.nseg, &scratch, block_);
       else
@@ -653,6 +751,60 @@ class Attention : public Mixer {
   }
 
  private:
+  // Norms, rotation, the values' blend and the store in one launch (qkv_prepare).
+  Tensor prepare(const Tensor& qkv, StepContext& ctx, CacheEntry& cache, GroupTables& tables) {
+    if (!cache.writable) throw EngineError("attention: unit or whole norms and mixed values need a cache of the layer's own");
+    Kernels::Prepare how;
+    if (unit_) {
+      how.norm = 2;
+      how.eps = unit_eps_;
+    } else if (q_norm_) {
+      how.norm = whole_ ? 3 : 1;
+      how.q_w = q_norm_->row_scale_weight();
+      how.k_w = k_norm_->row_scale_weight();
+      how.eps = q_norm_->eps();
+      if (!how.q_w || !how.k_w || k_norm_->eps() != how.eps) throw ConfigError("attention: these norms of q and k must be weighted row scales with one eps");
+    }
+    if (position_) {
+      how.inv_freq = position_->angle_frequencies();
+      if (!how.inv_freq || position_->magnitude() != 1.f || position_->pairs_neighbours())
+        throw ConfigError("attention: unit norms and mixed values are built with rotations of halves by computed angles");
+    }
+    const int64_t v_col = (int64_t)(nq_ + nkv_) * d_;
+    if (mix_ == 1) {
+      ctx.first_values = {qkv, v_col, nkv_, d_, dv_};
+    } else if (mix_ == 2) {
+      const HeadColumns& f = ctx.first_values;
+      if (!f.rows.data) throw EngineError("attention: no layer of this step kept its values for later ones");
+      if (f.heads * f.size != nkv_ * dv_) throw ConfigError("attention: " + std::to_string(nkv_ * dv_) + " values a token cannot be blended with " + std::to_string(f.heads * f.size));
+      how.share = &share_;
+      how.v0 = f.rows;
+      how.v0_col = f.first;
+      how.v0_d = f.stride;
+      how.v0_size = f.size;
+    }
+    return kernels.qkv_prepare(qkv, nq_, nkv_, d_, dk_, dv_, how, cache.k, cache.v, cache.page_size, ctx.positions, tables.slots);
+  }
+  // The learned table [classes, heads] as the kernels read it: a row a head, the largest distance first, padded at both ends.
+  void load_distances(const Tensor& table) {
+    const int64_t classes = table.dim(0), limit = 1 << 20;
+    if (classes < 1) throw EngineError("attention: a distance table of " + table.describe());
+    if (!(bias_max_ > (double)(classes / 2)) || bias_max_ > (double)limit)
+      throw ConfigError("attention: 'bias_max' " + std::to_string(bias_max_) + " must exceed half the distance table's " + std::to_string(classes) + " rows (and be at most " +
+                        std::to_string(limit) + ")");
+    far_ = 0;
+    while (distance_class(far_, classes, bias_max_) < classes - 1) ++far_;        // from here on every distance is of the last class
+    const std::vector<float> b = host_floats(table);
+    const int pad = kernels.distance_pad();
+    const int64_t width = (int64_t)far_ + 1 + 2 * pad;
+    std::vector<float> rows((size_t)(nq_ * width));
+    for (int h = 0; h < nq_; ++h)
+      for (int64_t i = 0; i < width; ++i) {
+        const int64_t n = std::min<int64_t>(std::max<int64_t>(far_ + pad - i, 0), far_);
+        rows[h * width + i] = b[(int64_t)distance_class(n, classes, bias_max_) * nq_ + h];
+      }
+    rel_ = float_tensor(std::move(rows)).view({(int64_t)nq_, width});
+  }
   // Norm, position encoding and store as separate steps, each sub-part through its own methods.
   Tensor unfused(const Tensor& qkv, StepContext& ctx, CacheEntry& cache, GroupTables& tables) {
     Kernels& k = kernels;
@@ -683,6 +835,12 @@ class Attention : public Mixer {
   bool exact_, own_kv_;
   int block_;                         // > 0: a row sees the keys of its own block of this many positions only
   bool gate_;                         // the heads' outputs times sigmoid(W_gate h)
+  bool head_gate_, unit_, whole_, bias_by_distance_;
+  int mix_;                           // 0: none, 1: the values that others mix with, 2: mixed with those
+  float unit_eps_;
+  double bias_max_;
+  int far_ = 0;                       // from this distance on the bias is the last class's
+  Tensor rel_, share_;
   std::unique_ptr<Norm> q_norm_, k_norm_;
   std::unique_ptr<PositionEncoding> position_;
   Tensor w_qkv_, w_o_, b_qkv_, sinks_;
@@ -726,14 +884,51 @@ class SwiGLU : public FeedForward {
   Tensor w_gate_up_, w_down_;
 };
 
+// down(max(up(x), 0)^2) without biases; the activation runs inside the first product's launch, on its rounded outputs.
+class SquaredRelu : public FeedForward {
+ public:
+  SquaredRelu(const PartSpec& s, Kernels& k) : FeedForward(k), hidden_(s.integer("hidden_size")), inter_(s.integer("intermediate_size")), run_(round_up(inter_, 64)) {}
+  std::vector<ParamDecl> params() const override { return {{"up_proj.weight", {inter_, hidden_}}, {"down_proj.weight", {hidden_, inter_}}}; }
+  void load(std::map<std::string, Tensor>& t) override {
+    w_up_ = pad_matrix(need(t, "up_proj.weight"), run_, hidden_);          // whole pairs of slabs; 0^2 adds nothing
+    w_down_ = pad_matrix(need(t, "down_proj.weight"), hidden_, run_);
+  }
+  int64_t gemm_floats(int64_t T) const { return std::max(kernels.gemm_workspace_floats(T, run_, hidden_), kernels.gemm_workspace_floats(T, hidden_, run_)); }
+  int64_t workspace_floats(HostStep& step) override {
+    int64_t T = 0;
+    for (int q : step.q_lens) T += q;
+    return gemm_floats(T);
+  }
+  Tensor forward(const Tensor& x, StepContext& ctx) override {
+    const int64_t n = gemm_floats(x.dim(0));
+    Tensor ws;
+    if (n) ws = ctx.workspace(n);
+    return kernels.gemm(kernels.gemm(x, w_up_, n ? &ws : nullptr, 1), w_down_, n ? &ws : nullptr);
+  }
+
+ private:
+  int64_t hidden_, inter_, run_;
+  Tensor w_up_, w_down_;
+};
+
+// A layer without a feed-forward names this kind; an arrangement that allows it never calls it.
+class NoFeedForward : public FeedForward {
+ public:
+  NoFeedForward(const PartSpec&, Kernels& k) : FeedForward(k) {}
+  Tensor forward(const Tensor&, StepContext&) override { throw EngineError("a layer without a feed-forward was asked to run one"); }
+};
+
 // x += mixer(norm(x)); x += ffn(norm(x)), carried as (hidden, residual) so that each add runs inside the
-// next norm (src/exec/dense_swiglu_decoder.rs:556-615 first layer, :740-813 others).
+// next norm (src/exec/dense_swiglu_decoder.rs:556-615 first layer, :740-813 others).  The residual is of the type the embedding
+// gave: elements, or the 32-bit stream.  A layer without a feed-forward ends after its mixer.
 class PreNormBlock : public Block {
  public:
   PreNormBlock(Kernels& k, std::unique_ptr<Mixer> mixer, std::unique_ptr<FeedForward> ffn, std::map<std::string, std::unique_ptr<Norm>> norms)
       : Block(k), mixer_(std::move(mixer)), ffn_(std::move(ffn)), norms_(std::move(norms)) {
+    has_ffn_ = dynamic_cast<NoFeedForward*>(ffn_.get()) == nullptr;
     for (const char* n : {"input", "post_mixer"})
-      if (!norms_.count(n)) throw ConfigError(std::string("a prenorm block needs the norms 'input' and 'post_mixer'; missing: ") + n);
+      if (!norms_.count(n) && (has_ffn_ || n == std::string("input")))
+        throw ConfigError(std::string("a prenorm block needs the norms 'input' and 'post_mixer'; missing: ") + n);
   }
   std::vector<std::pair<std::string, Part*>> children() override {
     std::vector<std::pair<std::string, Part*>> c = {{"mixer", mixer_.get()}, {"feed_forward", ffn_.get()}};
@@ -750,6 +945,7 @@ class PreNormBlock : public Block {
       normed = norms_["input"]->forward_add(hidden, residual);
     }
     const Tensor mixed = mixer_->forward(normed, ctx, cache);
+    if (!has_ffn_) return {mixed, residual};
     normed = norms_["post_mixer"]->forward_add(mixed, residual);
     return {ffn_->forward(normed, ctx), residual};
   }
@@ -758,6 +954,7 @@ class PreNormBlock : public Block {
   std::unique_ptr<Mixer> mixer_;
   std::unique_ptr<FeedForward> ffn_;
   std::map<std::string, std::unique_ptr<Norm>> norms_;
+  bool has_ffn_ = true;
 };
 
 // logits = x W^T without bias (src/exec/dense_swiglu_model.rs:976-984).  A head tied to the embedding is this
@@ -957,13 +1154,6 @@ class GatedLinearAttention : public Mixer {
   float root_, eps_;
   int64_t qk_ = 0, v_ = 0, gate_col_ = 0, decay_col_ = 0;
   Tensor w_in_, w_decay_up_, decay_bias_, out_norm_, w_o_;
-};
-
-// A layer without a feed-forward names this kind; an arrangement that allows it never calls it.
-class NoFeedForward : public FeedForward {
- public:
-  NoFeedForward(const PartSpec&, Kernels& k) : FeedForward(k) {}
-  Tensor forward(const Tensor&, StepContext&) override { throw EngineError("a layer without a feed-forward was asked to run one"); }
 };
 
 // A residual stream x in 32-bit, a norm before and after each sublayer, and (kind "sandwich_depth"; kind "sandwich" ends
@@ -1198,7 +1388,9 @@ class PairMean : public Mixer {
 // multiplies the gate and up outputs before their clamps, and the sum adds the experts' outputs as they are; score 2: the
 // weights are the softmax scores over all experts as they are), groups and keep_groups (the experts form that many equal runs of
 // neighbours, a group's score is its largest, and only experts of the best keep_groups can be chosen), weight_scale (on every
-// weight).  limit absent: nothing is clamped.
+// weight).  limit absent: nothing is clamped.  choice_correction (with score 1): a learned number an expert joins its score for the
+// choice of groups and experts, and not its weight; group_score 1: a group is worth the sum of its two largest (corrected)
+// scores.  A shared expert of experts that are not gated is W_down max(W_up h, 0)^2 like them.
 class RoutedExperts : public FeedForward {
  public:
   RoutedExperts(const PartSpec& s, Kernels& k)
@@ -1207,7 +1399,10 @@ class RoutedExperts : public FeedForward {
         gated_(s.integer("gated", 0) != 0), limit_((float)s.number("limit", 0.0)), slope_((float)s.number("glu_slope", 1.0)),
         shift_((float)s.number("up_shift", 0.0)), shared_(s.integer("shared_size", 0)), shared_limit_((float)s.number("shared_limit", 0.0)),
         score_((int)s.integer("score", 0)), weigh_input_(s.integer("weigh_input", 0) != 0), groups_((int)s.integer("groups", 1)),
-        keep_((int)s.integer("keep_groups", 1)), weight_scale_((float)s.number("weight_scale", 1.0)) {
+        keep_((int)s.integer("keep_groups", 1)), weight_scale_((float)s.number("weight_scale", 1.0)), corrected_(s.integer("choice_correction", 0) != 0),
+        group_score_((int)s.integer("group_score", 0)) {
+    if (corrected_ && (score_ != 1 || bias_ || weigh_input_)) throw ConfigError("experts: a correction of the choice is built for logistic scores without a router bias");
+    if (group_score_ < 0 || group_score_ > 1 || (group_score_ == 1 && !corrected_)) throw ConfigError("experts: 'group_score' is 0 (a group's largest) or, with a correction, 1 (the sum of its two largest)");
     if (score_ < 0 || score_ > 2)
       throw ConfigError("experts: 'score' is 0 (softmax, divided by the chosen sum), 1 (the logistic function of a chosen logit) or 2 (softmax as it is)");
     if (groups_ < 1 || experts_ % groups_ || keep_ < 1 || keep_ > groups_ || top_ > keep_ * (experts_ / groups_))
@@ -1217,8 +1412,7 @@ class RoutedExperts : public FeedForward {
     if (weigh_input_ && (!gated_ || shared_ > 0)) throw ConfigError("experts whose weights scale their inputs are built in the gated form, without a shared expert");
     if (experts_ < 1 || top_ < 1 || top_ > experts_) throw ConfigError("a mixture of " + std::to_string(experts_) + " experts cannot choose " + std::to_string(top_));
     if (gated_ && !(limit_ > 0.f)) throw ConfigError("gated experts need a positive 'limit'");
-    if (shared_ < 0 || (shared_ > 0 && (!gated_ || !(shared_limit_ > 0.f))))
-      throw ConfigError("a shared expert is built in the gated form, with a positive 'shared_limit'");
+    if (shared_ < 0 || (shared_ > 0 && gated_ && !(shared_limit_ > 0.f))) throw ConfigError("a gated shared expert needs a positive 'shared_limit'");
   }
   std::vector<ParamDecl> params() const override {
     std::vector<ParamDecl> p = {{"router.weight", {(int64_t)experts_, hidden_}}};
@@ -1227,13 +1421,17 @@ class RoutedExperts : public FeedForward {
       ParamDecl b{"router.bias", {(int64_t)experts_}, true, true, -0.5, 0.5};
       p.push_back(b);
     }
+    if (corrected_) {
+      ParamDecl c{"router.correction", {(int64_t)experts_}, true, true, -0.5, 0.5};
+      p.push_back(c);
+    }
     for (int e = 0; e < experts_; ++e) {
       if (gated_) p.push_back({"experts." + std::to_string(e) + ".gate_proj.weight", {inter_, hidden_}});
       p.push_back({"experts." + std::to_string(e) + ".up_proj.weight", {inter_, hidden_}});
       p.push_back({"experts." + std::to_string(e) + ".down_proj.weight", {hidden_, inter_}});
     }
     if (shared_ > 0) {
-      p.push_back({"shared.gate_proj.weight", {shared_, hidden_}});
+      if (gated_) p.push_back({"shared.gate_proj.weight", {shared_, hidden_}});
       p.push_back({"shared.up_proj.weight", {shared_, hidden_}});
       p.push_back({"shared.down_proj.weight", {hidden_, shared_}});
     }
@@ -1244,9 +1442,11 @@ class RoutedExperts : public FeedForward {
     const int64_t padded = round_up(inter_, 64);              // whole pairs of slabs, so that the tile product takes it
     std::vector<Tensor> up, down;
     if (bias_) router_bias_ = need(t, "router.bias");
+    if (corrected_) correction_ = need(t, "router.correction");
     if (shared_ > 0) {
       const int64_t sp = round_up(shared_, 64);
-      w_shared_in_ = stack_rows({pad_matrix(need(t, "shared.gate_proj.weight"), sp, hidden_), pad_matrix(need(t, "shared.up_proj.weight"), sp, hidden_)});
+      w_shared_in_ = pad_matrix(need(t, "shared.up_proj.weight"), sp, hidden_);
+      if (gated_) w_shared_in_ = stack_rows({pad_matrix(need(t, "shared.gate_proj.weight"), sp, hidden_), w_shared_in_});
       w_shared_down_ = pad_matrix(need(t, "shared.down_proj.weight"), hidden_, sp);
     }
     for (int e = 0; e < experts_; ++e) {
@@ -1264,28 +1464,32 @@ class RoutedExperts : public FeedForward {
     const int64_t pairs = x.dim(0) * top_;
     const Tensor* bias = bias_ ? &router_bias_ : nullptr;
     Tensor shared;
-    if (shared_ > 0) shared = k.gemm(k.moe_glu(k.gemm(x, w_shared_in_), shared_limit_, slope_, shift_), w_shared_down_);
+    if (shared_ > 0)
+      shared = k.gemm(gated_ ? k.moe_glu(k.gemm(x, w_shared_in_), shared_limit_, slope_, shift_) : k.gemm(x, w_shared_in_, nullptr, 1), w_shared_down_);
     const Tensor* extra = shared_ > 0 ? &shared : nullptr;
     // Few rows an expert: products over tiles of 16 rows that stream an expert's weights once a tile.  Many (prompts):
     // the rows are sorted by expert into blocks of 128 and go through the engine's tile product, every block with its
     // expert's matrix.  Both are launched from numbers on the GPU alone and give the same bits.
     if (pairs < (int64_t)kRowsAnExpertForTiles * experts_ || !k.gemm_grouped_takes(hidden_) || !k.gemm_grouped_takes(w_down_.dim(2))) {
-      const Kernels::MoePlan plan = k.moe_route_scored(x, router_, top_, weight_eps_, 16, bias, score_, groups_, keep_, weight_scale_);
+      const Kernels::MoePlan plan = route(x, 16, bias);
       if (weigh_input_)
         return k.moe_sum_unweighed(k.moe_down(k.moe_glu_weighed(k.moe_up_plain(x, w_up_, plan), limit_, slope_, shift_, plan), w_down_, plan), plan);
       const Tensor act = gated_ ? k.moe_glu(k.moe_up_plain(x, w_up_, plan), limit_, slope_, shift_) : k.moe_up(x, w_up_, plan);
       return k.moe_sum(k.moe_down(act, w_down_, plan), plan, extra);
     }
-    const Kernels::MoePlan plan = k.moe_route_scored(x, router_, top_, weight_eps_, 128, bias, score_, groups_, keep_, weight_scale_);
-    Tensor act = k.gemm_grouped(k.gather_rows(x, plan.row_token), w_up_, plan.tile_expert);
+    const Kernels::MoePlan plan = route(x, 128, bias);
+    Tensor act = k.gemm_grouped(k.gather_rows(x, plan.row_token), w_up_, plan.tile_expert, gated_ ? 0 : 1);
     if (weigh_input_) return k.moe_sum_unweighed(k.gemm_grouped(k.moe_glu_weighed(act, limit_, slope_, shift_, plan), w_down_, plan.tile_expert), plan);
     if (gated_) act = k.moe_glu(act, limit_, slope_, shift_);
-    else k.relu_square(act);
     return k.moe_sum(k.gemm_grouped(act, w_down_, plan.tile_expert), plan, extra);
   }
   static constexpr int kRowsAnExpertForTiles = 32;
 
  private:
+  Kernels::MoePlan route(const Tensor& x, int tile_rows, const Tensor* bias) {
+    if (corrected_) return kernels.moe_route_corrected(x, router_, correction_, top_, tile_rows, groups_, keep_, group_score_, weight_scale_);
+    return kernels.moe_route_scored(x, router_, top_, weight_eps_, tile_rows, bias, score_, groups_, keep_, weight_scale_);
+  }
   int64_t hidden_, inter_;
   int experts_, top_;
   float weight_eps_;
@@ -1297,7 +1501,9 @@ class RoutedExperts : public FeedForward {
   bool weigh_input_;       // a weight scales what its expert reads (the gate and up outputs before their clamps), not what it gives
   int groups_, keep_;      // experts of the best keep_ of groups_ equal groups can be chosen
   float weight_scale_;
-  Tensor router_, router_bias_, w_up_, w_down_, w_shared_in_, w_shared_down_;
+  bool corrected_;         // a learned number an expert joins its score for the choice alone
+  int group_score_;        // 0: a group is worth its largest score, 1: the sum of its two largest
+  Tensor router_, router_bias_, correction_, w_up_, w_down_, w_shared_in_, w_shared_down_;
 };
 
 // Mixer and feed-forward side by side on a residual stream x in 32-bit: x <- x + (mixer(norm_mixer_in(x)) +
@@ -1827,6 +2033,8 @@ void register_standard_parts() {
                                        std::map<std::string, std::unique_ptr<Norm>> n, const std::map<std::string, double>& numbers) {
       return std::unique_ptr<Block>(new HyperStreamsBlock(k, std::move(m), std::move(f), std::move(n), numbers));
     });
+    register_part("embedding", "token_embedding_bigram", factory<BigramEmbedding>());
+    register_part("feed_forward", "squared_relu", factory<SquaredRelu>());
     register_part("norm", "rmsnorm", factory<RMSNorm>());
     register_part("position", "rotary", factory<Rotary>());
     register_part("mixer", "attention", factory<Attention>());

@@ -36,6 +36,8 @@ struct HostArray {
 // What the host knows of a step before anything is uploaded.
 struct HostStep {
   std::vector<int> q_lens, starts, k_lens, state_slots;
+  std::vector<int32_t> ids;       // the step's tokens, sequence after sequence
+  std::vector<int32_t> before;    // per sequence: the token before its first one of this step, -1 at a request's start
   int k_len_bound = 0;            // no k_len is larger
   bool frozen = false;            // the step is recorded for replay: launches must cover k_len_bound keys
   std::map<std::string, std::shared_ptr<void>> memo;   // parts keep what they derive once per step here
@@ -47,6 +49,13 @@ struct GroupTables {
   int window = 0;
 };
 
+// Columns of a tensor that hold heads: head h's entries are the columns first + h * stride .. + size.
+struct HeadColumns {
+  Tensor rows;
+  int64_t first = 0;
+  int heads = 0, stride = 0, size = 0;
+};
+
 struct StepContext {
   Kernels* kernels = nullptr;
   int num_tokens = 0, num_seqs = 0;
@@ -55,6 +64,7 @@ struct StepContext {
   HostStep* host = nullptr;
   std::map<std::string, Tensor> inputs;              // the arrays parts asked for, on the GPU
   std::map<std::string, Tensor> carry;               // what a part leaves for later parts of the same step (empty at its start)
+  HeadColumns first_values;                          // the values that the step's first layer that mixes values projected
   std::function<Tensor(int64_t)> workspace;           // float32 scratch of at least that many elements
 };
 
@@ -107,7 +117,8 @@ class Norm : public Part {
  public:
   using Part::Part;
   virtual Tensor forward(const Tensor& x) = 0;
-  // residual += x in place (the sum in 32-bit, stored rounded); returns the norm of the unrounded sum.
+  // residual += x in place (the sum in 32-bit, stored rounded, or as it is where the residual is a 32-bit stream); returns the
+  // norm of the unrounded sum.
   virtual Tensor forward_add(const Tensor& x, Tensor& residual) = 0;
   // A norm that is y = x * rsqrt(mean(x^2) + eps) * w says so; a mixer may then run it inside a launch of its own.
   virtual const Tensor* row_scale_weight() const { return nullptr; }

@@ -163,6 +163,7 @@ ModelRunner::Layout ModelRunner::layout(const std::vector<StepEntry>& entries, c
     host.starts.push_back(cache.length(e.id));
     host.k_lens.push_back(cache.length(e.id) + n);
     host.state_slots.push_back(cache.state_slot(e.id));
+    host.before.push_back(cache.token(e.id, host.starts.back() - 1));
     T += n;
   }
   for (int i = 0; i < pad; ++i) {
@@ -170,6 +171,7 @@ ModelRunner::Layout ModelRunner::layout(const std::vector<StepEntry>& entries, c
     host.starts.push_back(0);
     host.k_lens.push_back(1);
     host.state_slots.push_back(0);
+    host.before.push_back(-1);
   }
   const int longest = *std::max_element(host.k_lens.begin(), host.k_lens.end());
   if (longest > spec.max_positions)
@@ -203,6 +205,7 @@ ModelRunner::Layout ModelRunner::layout(const std::vector<StepEntry>& entries, c
     slots.data.push_back(host.state_slots[s]);
   }
   ids.shape = positions.shape = {T};
+  host.ids = ids.data;
   cu_q.shape = {S + 1};
   k_len.shape = slots.shape = {S};
   want.shape = {(int64_t)want.data.size()};

@@ -42,11 +42,22 @@
 
 static int device_cus();      // compute units of the current device (defined with the host code below)
 
+// How a product's sums leave a kernel: whether rows take 16-byte (8-byte) stores, and an activation on the rounded sums.
+#define OUT_VEC 1
+#define OUT_SQUARED_RELU 2            // max(., 0)^2
+
 __device__ __forceinline__ void store_out4(elem_t* out, int64_t ldo, int m, int n, int M, int N, f32x4 v,
-                                           bool vec_ok) {
+                                           int form) {
   if (m >= M || n >= N) return;
+  if (form & OUT_SQUARED_RELU) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float r = fmaxf(round_to_elem(v[i]), 0.f);
+      v[i] = r * r;
+    }
+  }
   elem_t* p = out + (int64_t)m * ldo + n;
-  if (vec_ok && n + 3 < N) {
+  if ((form & OUT_VEC) && n + 3 < N) {
 #ifdef VK_F32
     *reinterpret_cast<f32x4*>(p) = v;
 #else
@@ -68,7 +79,7 @@ template <int MT, int W>
 __global__ __launch_bounds__(64 * SK_WAVES) void gemm_skinny_kernel(elem_t* __restrict__ out,
                                                                     const elem_t* __restrict__ act,
                                                                     const elem_t* __restrict__ w, int M, int N, int K,
-                                                                    int64_t lda, int64_t ldo, int out_vec_ok) {
+                                                                    int64_t lda, int64_t ldo, int out_form) {
   static_assert(KC_SLABS % W == 0, "the window must divide a chunk");
   __shared__ f32x4 part[SK_WAVES][MT][64];
 
@@ -137,7 +148,7 @@ __global__ __launch_bounds__(64 * SK_WAVES) void gemm_skinny_kernel(elem_t* __re
     }
     __syncthreads();
   }
-  if (wave < MT) store_out4(out, ldo, wave * 16 + r16, n0 + 4 * kg, M, N, total, out_vec_ok);
+  if (wave < MT) store_out4(out, ldo, wave * 16 + r16, n0 + 4 * kg, M, N, total, out_form);
 }
 
 // ---------------------------------------------------------------- streaming
@@ -153,7 +164,7 @@ template <int MT, int W, int RC, int NT, int NW = SK_WAVES>
 __global__ __launch_bounds__(64 * NW) void gemm_stream_kernel(elem_t* __restrict__ out,
                                                                     const elem_t* __restrict__ act,
                                                                     const elem_t* __restrict__ w, int M, int N, int K,
-                                                                    int64_t lda, int64_t ldo, int out_vec_ok) {
+                                                                    int64_t lda, int64_t ldo, int out_form) {
   // NT: 16-row weight tiles per workgroup.  With several activation tiles every workgroup reads all
   // activations once, M * K elements beside its 16 * NT * K weights: more weight rows per workgroup
   // keep that traffic, which comes from the second-level cache, in proportion.
@@ -259,7 +270,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_stream_kernel(elem_t* __restrict
       for (int base = 0; base < nchunks; base += NW) round(base, 0);
     }
     if (wave < NT * MT)
-      store_out4(out, ldo, (wave % MT) * 16 + r16, (tile * NT + wave / MT) * 16 + 4 * kg, M, N, total, out_vec_ok);
+      store_out4(out, ldo, (wave % MT) * 16 + r16, (tile * NT + wave / MT) * 16 + 4 * kg, M, N, total, out_form);
   }
 }
 
@@ -274,7 +285,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_stream_swiglu_kernel(elem_t* __r
                                                                            const elem_t* __restrict__ act,
                                                                            const elem_t* __restrict__ w, int M, int I,
                                                                            int K, int64_t lda, int64_t ldo,
-                                                                           int out_vec_ok) {
+                                                                           int out_form) {
   static_assert(KC_SLABS % W == 0, "the window must divide a chunk");
   static_assert(MT * RC <= 2, "two chunk tiles of activations stay in registers: two tiles of a chunk or two chunks of a tile");
   __shared__ f32x4 part[2][RC][NW][2 * MT][64];      // two sets, used in turn: one barrier per tile
@@ -360,7 +371,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_stream_swiglu_kernel(elem_t* __r
       y.y = (g[1] * (1.0f / (1.0f + expf(-g[1])))) * u[1];
       y.z = (g[2] * (1.0f / (1.0f + expf(-g[2])))) * u[2];
       y.w = (g[3] * (1.0f / (1.0f + expf(-g[3])))) * u[3];
-      store_out4(out, ldo, wave * 16 + r16, tile * 16 + 4 * kg, M, I, y, out_vec_ok);
+      store_out4(out, ldo, wave * 16 + r16, tile * 16 + 4 * kg, M, I, y, out_form);
     }
     parity ^= 1;
   }
@@ -377,7 +388,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_stream_swiglu_kernel(elem_t* __r
 template <int FN, int FM>
 __global__ __launch_bounds__(256) void gemm_tiled_kernel(elem_t* __restrict__ out, const elem_t* __restrict__ act,
                                                          const elem_t* __restrict__ w, int M, int N, int K,
-                                                         int64_t lda, int64_t ldo, int out_vec_ok) {
+                                                         int64_t lda, int64_t ldo, int out_form) {
   constexpr int BN = 32 * FN, BM = 32 * FM;
   constexpr int W_BYTES = BN * T_ROWB, A_BYTES = BM * T_ROWB, BUF_BYTES = W_BYTES + A_BYTES;
   extern __shared__ __attribute__((aligned(16))) unsigned char lds[];   // [buffer][w tile, act tile]
@@ -477,12 +488,12 @@ __global__ __launch_bounds__(256) void gemm_tiled_kernel(elem_t* __restrict__ ou
 #pragma unroll
     for (int j = 0; j < FM; ++j)
       store_out4(out, ldo, m_blk + wm * 16 * FM + j * 16 + r16, n_blk + wn * 16 * FN + i * 16 + 4 * kg, M, N,
-                 total[i][j], out_vec_ok);
+                 total[i][j], out_form);
 }
 
 template <int FN, int FM>
 static int launch_tiled(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K, int64_t lda, int64_t ldo,
-                        int vec_ok, hipStream_t st) {
+                        int form, hipStream_t st) {
   constexpr int BN = 32 * FN, BM = 32 * FM;
   const size_t smem = 2 * (size_t)(BN + BM) * T_ROWB;
   static bool configured = false;
@@ -494,7 +505,7 @@ static int launch_tiled(elem_t* out, const elem_t* act, const elem_t* w, int M, 
   }
   dim3 grid((N + BN - 1) / BN, (M + BM - 1) / BM);
   VK_REQUIRE(grid.y <= 65535, "gemm: too many rows (%d)", M);
-  gemm_tiled_kernel<FN, FM><<<grid, 256, smem, st>>>(out, act, w, M, N, K, lda, ldo, vec_ok);
+  gemm_tiled_kernel<FN, FM><<<grid, 256, smem, st>>>(out, act, w, M, N, K, lda, ldo, form);
   return vk_check_launch("gemm_tiled");
 }
 
@@ -560,7 +571,7 @@ __device__ __forceinline__ void wait_vmcnt_n() {             // vmcnt(N_), N_ be
 template <int S, bool WHOLE, bool SWIGLU, int FNW = 4, int PFD = 0>
 __global__ __launch_bounds__(256, 2) void gemm_pipe_kernel(elem_t* __restrict__ out, const elem_t* __restrict__ act,
                                                         const elem_t* __restrict__ w, int M, int N, int K,
-                                                        int64_t lda, int64_t ldo, int out_vec_ok, int band_w,
+                                                        int64_t lda, int64_t ldo, int out_form, int band_w,
                                                         const int32_t* __restrict__ block_weights, int64_t weights_stride) {
   static_assert(FNW >= 2 && FNW <= 5 && (FNW == 4 || !SWIGLU), "two to five weight fragments per wave; four with SwiGLU");
   static_assert(PFD == 0 || FNW == 2 || FNW == 4, "the touch-ahead wants a wave's 64 rows to be of one kind");
@@ -760,7 +771,7 @@ __global__ __launch_bounds__(256, 2) void gemm_pipe_kernel(elem_t* __restrict__ 
         y.y = (g.y * (1.0f / (1.0f + expf(-g.y)))) * u.y;
         y.z = (g.z * (1.0f / (1.0f + expf(-g.z)))) * u.z;
         y.w = (g.w * (1.0f / (1.0f + expf(-g.w)))) * u.w;
-        store_out4(out, ldo, m_blk + wm * 64 + j * 16 + r16, n_blk + i * 16 + 4 * kg, M, N, y, out_vec_ok);
+        store_out4(out, ldo, m_blk + wm * 64 + j * 16 + r16, n_blk + i * 16 + 4 * kg, M, N, y, out_form);
       }
     }
     return;
@@ -770,7 +781,7 @@ __global__ __launch_bounds__(256, 2) void gemm_pipe_kernel(elem_t* __restrict__ 
 #pragma unroll
     for (int j = 0; j < 4; ++j)
       store_out4(out, ldo, m_blk + wm * 64 + j * 16 + r16, n_blk + wn * 16 * FNW + i * 16 + 4 * kg, M, N, total[i][j],
-                 out_vec_ok);
+                 out_form);
 }
 
 // Column blocks of a band in the tile kernel (0: no bands).  64: the 512 workgroups that run at a time
@@ -783,7 +794,7 @@ static const int pipe_band_blocks = 64;
 
 template <int S, bool SWIGLU = false, int FNW = 4>
 static int launch_pipe(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K, int64_t lda, int64_t ldo,
-                       int vec_ok, hipStream_t st, const int32_t* block_weights = nullptr, int64_t weights_stride = 0) {
+                       int form, hipStream_t st, const int32_t* block_weights = nullptr, int64_t weights_stride = 0) {
   constexpr int BN = SWIGLU ? 64 : 32 * FNW;                         // output columns of a workgroup
   const size_t smem = (size_t)S * (32 * FNW + 128) * T_ROWB;         // also holds the 32 KB that SWIGLU passes between waves
   static bool configured = false;
@@ -806,12 +817,12 @@ static int launch_pipe(elem_t* out, const elem_t* act, const elem_t* w, int M, i
         (void)hipFuncSetAttribute((const void*)gemm_pipe_kernel<S, true, SWIGLU, FNW, 4>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
         touched = true;
       }
-      gemm_pipe_kernel<S, true, SWIGLU, FNW, 4><<<grid, 256, smem, st>>>(out, act, w, M, N, K, lda, ldo, vec_ok, band_w, block_weights, weights_stride);
+      gemm_pipe_kernel<S, true, SWIGLU, FNW, 4><<<grid, 256, smem, st>>>(out, act, w, M, N, K, lda, ldo, form, band_w, block_weights, weights_stride);
       return vk_check_launch("gemm_pipe");
     }
   }
-  if (K % KC == 0) gemm_pipe_kernel<S, true, SWIGLU, FNW><<<grid, 256, smem, st>>>(out, act, w, M, N, K, lda, ldo, vec_ok, band_w, block_weights, weights_stride);
-  else gemm_pipe_kernel<S, false, SWIGLU, FNW><<<grid, 256, smem, st>>>(out, act, w, M, N, K, lda, ldo, vec_ok, band_w, block_weights, weights_stride);
+  if (K % KC == 0) gemm_pipe_kernel<S, true, SWIGLU, FNW><<<grid, 256, smem, st>>>(out, act, w, M, N, K, lda, ldo, form, band_w, block_weights, weights_stride);
+  else gemm_pipe_kernel<S, false, SWIGLU, FNW><<<grid, 256, smem, st>>>(out, act, w, M, N, K, lda, ldo, form, band_w, block_weights, weights_stride);
   return vk_check_launch("gemm_pipe");
 }
 
@@ -844,7 +855,7 @@ __device__ __forceinline__ void mid_load_to_lds16(const elem_t* src, unsigned ch
 template <int MT, int KH, bool SWIGLU = false, int GT = 4>
 __global__ __launch_bounds__(512) void gemm_mid_kernel(elem_t* __restrict__ out, const elem_t* __restrict__ act,
                                                        const elem_t* __restrict__ w, int M, int N, int K,
-                                                       int64_t lda, int64_t ldo, int out_vec_ok) {
+                                                       int64_t lda, int64_t ldo, int out_form) {
   static_assert(!SWIGLU || KH == 1, "the SwiGLU epilogue pairs the waves of one chunk");
   static_assert(GT == 4 || (SWIGLU && GT >= 2 && GT < 4), "fewer gate tiles only with the SwiGLU epilogue");
   constexpr int NTW = 8 / KH;                       // waves side by side along the weight rows
@@ -998,21 +1009,21 @@ __global__ __launch_bounds__(512) void gemm_mid_kernel(elem_t* __restrict__ out,
           y.y = (g[1] * (1.0f / (1.0f + expf(-g[1])))) * u[1];
           y.z = (g[2] * (1.0f / (1.0f + expf(-g[2])))) * u[2];
           y.w = (g[3] * (1.0f / (1.0f + expf(-g[3])))) * u[3];
-          store_out4(out, ldo, row0 + mt * 16 + r16, out_col0 + 4 * kg, M, N, y, out_vec_ok);
+          store_out4(out, ldo, row0 + mt * 16 + r16, out_col0 + 4 * kg, M, N, y, out_form);
         }
       }
       return;
     }
 #pragma unroll
     for (int mt = 0; mt < MT; ++mt)
-      store_out4(out, ldo, row0 + mt * 16 + r16, out_col0 + 4 * kg, M, N, total[mt], out_vec_ok);
+      store_out4(out, ldo, row0 + mt * 16 + r16, out_col0 + 4 * kg, M, N, total[mt], out_form);
   }
 }
 
 // N: weight rows, or with SWIGLU the gate rows (and as many up rows after them).
 template <int MT, int KH, bool SWIGLU = false, int GT = 4>
 static int launch_mid(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K, int64_t lda, int64_t ldo,
-                      int vec_ok, hipStream_t st) {
+                      int form, hipStream_t st) {
   constexpr int NTW = 8 / KH;
   constexpr int COLS = SWIGLU ? 16 * GT : 16 * NTW; // output columns of a workgroup
   const size_t smem = (size_t)2 * KH * 16 * MT * (MID_QS * 64) + (size_t)(KH - 1) * NTW * MT * 64 * sizeof(f32x4);
@@ -1025,7 +1036,7 @@ static int launch_mid(elem_t* out, const elem_t* act, const elem_t* w, int M, in
   // Blocks of 16 MT rows side by side: those of a weight tile run at about the same time, and on the same
   // chip part when the grid's width is a multiple of eight, so that all but one find it in its cache.
   const dim3 grid((N + COLS - 1) / COLS, (M + 16 * MT - 1) / (16 * MT));
-  gemm_mid_kernel<MT, KH, SWIGLU, GT><<<grid, 512, smem, st>>>(out, act, w, M, N, K, lda, ldo, vec_ok);
+  gemm_mid_kernel<MT, KH, SWIGLU, GT><<<grid, 512, smem, st>>>(out, act, w, M, N, K, lda, ldo, form);
   return vk_check_launch("gemm_mid");
 }
 
@@ -1092,7 +1103,7 @@ __global__ __launch_bounds__(64 * NTW) void gemm_split_kernel(f32x4* __restrict_
 template <int MT>
 __global__ __launch_bounds__(256) void gemm_split_reduce_kernel(elem_t* __restrict__ out, const f32x4* __restrict__ partial,
                                                                 int M, int N, int64_t ldo, int nchunks, int ntiles16,
-                                                                int up_tiles, int out_vec_ok) {
+                                                                int up_tiles, int out_form) {
   const int64_t t = (int64_t)blockIdx.x * 256 + threadIdx.x;
   const int lane = (int)(t & 63), mt = (int)((t >> 6) % MT);
   const int tile = (int)(t / (64 * MT));
@@ -1129,12 +1140,12 @@ __global__ __launch_bounds__(256) void gemm_split_reduce_kernel(elem_t* __restri
     y.z = (g[2] * (1.0f / (1.0f + expf(-g[2])))) * u[2];
     y.w = (g[3] * (1.0f / (1.0f + expf(-g[3])))) * u[3];
   }
-  store_out4(out, ldo, mt * 16 + r16, tile * 16 + 4 * kg, M, N, y, out_vec_ok);
+  store_out4(out, ldo, mt * 16 + r16, tile * 16 + 4 * kg, M, N, y, out_form);
 }
 
 template <int MT>
 static int launch_split(elem_t* out, const elem_t* act, const elem_t* w, int M, int rows, int K, int64_t lda, int64_t ldo,
-                        int swiglu, float* workspace, int vec_ok, hipStream_t st) {
+                        int swiglu, float* workspace, int form, hipStream_t st) {
   const int ntiles16 = (rows + 15) / 16, nchunks = K / KC;
   f32x4* partial = reinterpret_cast<f32x4*>(workspace);
   // Eight waves a workgroup where that still leaves two workgroups or more per compute unit, else four
@@ -1147,7 +1158,7 @@ static int launch_split(elem_t* out, const elem_t* act, const elem_t* w, int M, 
   const int out_tiles = swiglu ? up_tiles : ntiles16;
   const int64_t threads = (int64_t)out_tiles * MT * 64;
   gemm_split_reduce_kernel<MT><<<(unsigned)((threads + 255) / 256), 256, 0, st>>>(out, partial, M, swiglu ? rows / 2 : rows, ldo,
-                                                                                  nchunks, ntiles16, up_tiles, vec_ok);
+                                                                                  nchunks, ntiles16, up_tiles, form);
   return vk_check_launch("gemm_split");
 }
 #endif
@@ -1273,19 +1284,31 @@ static int pipe_fragments_by_rounds(int M, int N) {
 
 extern "C" {
 
+// The element type's activation code in a product's entry point: 0 none, 1 the square of max(., 0) on the rounded sums (the bits
+// of the plain product followed by vk_moe_relu_square).
+static int out_form_of(const elem_t* out, int64_t ldo, int activation) {
+  return ((ldo % 4 == 0) && ((uintptr_t)out % 16 == 0) ? OUT_VEC : 0) | (activation == 1 ? OUT_SQUARED_RELU : 0);
+}
+
 // A grouped product through the tile kernel: rows in blocks of 128, block b multiplied by the weight matrix
 // block_weights[b] of several [N, K] matrices that lie weights_stride elements apart (negative: the block is skipped and
 // its output rows are left as they are).  K in whole pairs of slabs (128 bytes of a row).  The same bits as vk_gemm gives
 // for the same rows and matrix.
-int vk_gemm_grouped(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K, int64_t lda, int64_t ldo,
-                    const int32_t* block_weights, int64_t weights_stride, hipStream_t st) {
+int vk_gemm_grouped_act(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K, int64_t lda, int64_t ldo,
+                        const int32_t* block_weights, int64_t weights_stride, int activation, hipStream_t st) {
+  VK_REQUIRE(activation == 0 || activation == 1, "grouped gemm: unknown activation %d", activation);
   VK_REQUIRE(M >= 0 && N > 0 && K > 0 && M % 128 == 0, "grouped gemm: bad sizes M=%d N=%d K=%d (rows in blocks of 128)", M, N, K);
   VK_REQUIRE(K % (2 * VK_SLAB) == 0, "grouped gemm: K=%d must be a multiple of %d", K, 2 * VK_SLAB);
   VK_REQUIRE(lda >= K && lda % VK_VEC == 0 && ldo >= N, "grouped gemm: bad row strides");
   VK_REQUIRE(((uintptr_t)act % 16) == 0 && ((uintptr_t)w % 16) == 0 && block_weights != nullptr && weights_stride % VK_VEC == 0,
              "grouped gemm: operands must be 16-byte aligned");
   if (M == 0) return 0;
-  return launch_pipe<2>(out, act, w, M, N, K, lda, ldo, (ldo % 4 == 0) && ((uintptr_t)out % 16 == 0), st, block_weights, weights_stride);
+  return launch_pipe<2>(out, act, w, M, N, K, lda, ldo, out_form_of(out, ldo, activation), st, block_weights, weights_stride);
+}
+
+int vk_gemm_grouped(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K, int64_t lda, int64_t ldo,
+                    const int32_t* block_weights, int64_t weights_stride, hipStream_t st) {
+  return vk_gemm_grouped_act(out, act, w, M, N, K, lda, ldo, block_weights, weights_stride, 0, st);
 }
 
 // kernel: 0 = choose by size, 1 = skinny (M <= 64), 2 = tiled (pipelined if K allows), 3 = tiled through
@@ -1294,8 +1317,9 @@ int vk_gemm_grouped(elem_t* out, const elem_t* act, const elem_t* w, int M, int 
 // (17 to 512 rows, in blocks of 64 rows), 11 = skinny with two activation tiles resident in registers (17 to
 // 32 rows of 16-bit elements, K <= 4096), 12 = as 9 in blocks of 32 rows, 13, 15 and 16 = pipelined with 64, 96
 // and 160 weight rows per workgroup (14 is the callers' name for the route through chunk sums); for measurements and tests.  The result does not depend on the choice.
-int vk_gemm(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K, int64_t lda, int64_t ldo,
-            int kernel, hipStream_t st) {
+static int gemm_launch(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K, int64_t lda, int64_t ldo,
+                       int kernel, int activation, hipStream_t st) {
+  VK_REQUIRE(activation == 0 || activation == 1, "gemm: unknown activation %d", activation);
   VK_REQUIRE(M >= 0 && N > 0 && K > 0, "gemm: bad sizes M=%d N=%d K=%d", M, N, K);
   VK_REQUIRE(K % VK_VEC == 0, "gemm: K=%d must be a multiple of %d for this element type", K, VK_VEC);
   VK_REQUIRE(lda >= K && lda % VK_VEC == 0, "gemm: activation row stride %lld must be >= K and a multiple of %d",
@@ -1304,29 +1328,29 @@ int vk_gemm(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K
   VK_REQUIRE(((uintptr_t)act % 16) == 0 && ((uintptr_t)w % 16) == 0, "gemm: operands must be 16-byte aligned");
   VK_REQUIRE(kernel >= 0 && kernel <= 16 && kernel != 14, "gemm: unknown kernel %d", kernel);
   if (M == 0) return 0;
-  const int vec_ok = (ldo % 4 == 0) && ((uintptr_t)out % 16 == 0);
+  const int form = out_form_of(out, ldo, activation);
   const bool by_size = kernel == 0;
   if (kernel == 0) kernel = choose_gemm_kernel(M, N, K);
   if (kernel == 12) {      // 32 weight rows per workgroup, four chunks in work, blocks of 32 rows
     VK_REQUIRE(M > 16 && M <= 512 && K % KC == 0, "gemm: the mid kernel takes 17 to 512 rows and K a multiple of %d", KC);
-    return launch_mid<2, 4>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
+    return launch_mid<2, 4>(out, act, w, M, N, K, lda, ldo, form, st);
   }
   if (kernel >= 8 && kernel <= 10) {
     VK_REQUIRE(M > 16 && M <= 512 && K % KC == 0, "gemm: the mid kernel takes 17 to 512 rows and K a multiple of %d", KC);
     const int mt = M > 64 ? 4 : (M + 15) / 16;       // more than 64 rows: blocks of 64
     if (kernel == 10) {     // 128 weight rows per workgroup, every wave all chunks of its tile
-      if (mt == 2) return launch_mid<2, 1>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
-      return launch_mid<4, 1>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
+      if (mt == 2) return launch_mid<2, 1>(out, act, w, M, N, K, lda, ldo, form, st);
+      return launch_mid<4, 1>(out, act, w, M, N, K, lda, ldo, form, st);
     }
     if (kernel == 8) {      // 64 weight rows per workgroup, two chunks in work
-      if (mt == 2) return launch_mid<2, 2>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
-      if (mt == 3) return launch_mid<3, 2>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
-      return launch_mid<4, 2>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
+      if (mt == 2) return launch_mid<2, 2>(out, act, w, M, N, K, lda, ldo, form, st);
+      if (mt == 3) return launch_mid<3, 2>(out, act, w, M, N, K, lda, ldo, form, st);
+      return launch_mid<4, 2>(out, act, w, M, N, K, lda, ldo, form, st);
     }
     // 32 weight rows per workgroup, four chunks in work
-    if (mt == 2) return launch_mid<2, 4>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
-    if (mt == 3) return launch_mid<3, 4>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
-    return launch_mid<4, 4>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
+    if (mt == 2) return launch_mid<2, 4>(out, act, w, M, N, K, lda, ldo, form, st);
+    if (mt == 3) return launch_mid<3, 4>(out, act, w, M, N, K, lda, ldo, form, st);
+    return launch_mid<4, 4>(out, act, w, M, N, K, lda, ldo, form, st);
   }
   if (kernel == 11)
     VK_REQUIRE(M > 16 && M <= 32 && K % KC == 0 && K <= SK_WAVES * KC && sizeof(elem_t) == 2,
@@ -1349,7 +1373,7 @@ int vk_gemm(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K
     }                                                                                                     \
     const unsigned groups = (unsigned)((N + 16 * NT - 1) / (16 * NT));                                    \
     gemm_stream_kernel<MT, W, RC, NT, NW><<<groups < (unsigned)resident ? groups : (unsigned)resident,    \
-                                             64 * NW, 0, st>>>(out, act, w, M, N, K, lda, ldo, vec_ok);   \
+                                             64 * NW, 0, st>>>(out, act, w, M, N, K, lda, ldo, form);   \
   } while (0)
 #define ST(MT, W, RC, NT) STW(MT, W, RC, NT, SK_WAVES)
       if (mt == 1) {
@@ -1393,7 +1417,7 @@ int vk_gemm(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K
 #undef STW
       return vk_check_launch("gemm_stream");
     }
-#define SK(MT, W) gemm_skinny_kernel<MT, W><<<grid, 64 * SK_WAVES, 0, st>>>(out, act, w, M, N, K, lda, ldo, vec_ok)
+#define SK(MT, W) gemm_skinny_kernel<MT, W><<<grid, 64 * SK_WAVES, 0, st>>>(out, act, w, M, N, K, lda, ldo, form)
     // Few weight rows leave one workgroup per compute unit: a deeper window keeps its memory pipe full.
     if (mt == 1) { if (N <= 8192) SK(1, 16); else SK(1, 8); }
     else if (mt == 2) SK(2, 8);
@@ -1403,23 +1427,34 @@ int vk_gemm(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K
     return vk_check_launch("gemm_skinny");
   }
   const bool k_whole = K % (2 * VK_SLAB) == 0;
-  if (kernel == 3) return launch_tiled<4, 4>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
-  if (kernel == 4 && k_whole) return launch_pipe<2>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
-  if (kernel == 5 && k_whole) return launch_pipe<3>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
-  if (kernel == 6 && k_whole) return launch_pipe<4>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
+  if (kernel == 3) return launch_tiled<4, 4>(out, act, w, M, N, K, lda, ldo, form, st);
+  if (kernel == 4 && k_whole) return launch_pipe<2>(out, act, w, M, N, K, lda, ldo, form, st);
+  if (kernel == 5 && k_whole) return launch_pipe<3>(out, act, w, M, N, K, lda, ldo, form, st);
+  if (kernel == 6 && k_whole) return launch_pipe<4>(out, act, w, M, N, K, lda, ldo, form, st);
   // Two stages of 32 KB leave room for two workgroups per compute unit, which hides more latency than a third stage.
   if (k_whole) {
     // No more 128 x 128 tiles than compute units: 64 weight rows a workgroup, twice as many of them
     // (512 rows, 4096 x 12288: 163 -> 145 us; a workgroup alone on its compute unit is bound by what one
     // compute unit can read, whatever the number of stages).
     const int64_t tiles = (int64_t)((N + 127) / 128) * ((M + 127) / 128);
-    if (kernel == 13 || (by_size && tiles <= device_cus())) return launch_pipe<2, false, 2>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
+    if (kernel == 13 || (by_size && tiles <= device_cus())) return launch_pipe<2, false, 2>(out, act, w, M, N, K, lda, ldo, form, st);
     const int fragments = kernel == 15 ? 3 : (kernel == 16 ? 5 : (by_size ? pipe_fragments_by_rounds(M, N) : 4));
-    if (fragments == 3) return launch_pipe<2, false, 3>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
-    if (fragments == 5) return launch_pipe<2, false, 5>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
-    return launch_pipe<2>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
+    if (fragments == 3) return launch_pipe<2, false, 3>(out, act, w, M, N, K, lda, ldo, form, st);
+    if (fragments == 5) return launch_pipe<2, false, 5>(out, act, w, M, N, K, lda, ldo, form, st);
+    return launch_pipe<2>(out, act, w, M, N, K, lda, ldo, form, st);
   }
-  return launch_tiled<4, 4>(out, act, w, M, N, K, lda, ldo, vec_ok, st);
+  return launch_tiled<4, 4>(out, act, w, M, N, K, lda, ldo, form, st);
+}
+
+int vk_gemm(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K, int64_t lda, int64_t ldo,
+            int kernel, hipStream_t st) {
+  return gemm_launch(out, act, w, M, N, K, lda, ldo, kernel, 0, st);
+}
+
+// vk_gemm (the kernel chosen by size) with an activation on the outputs.
+int vk_gemm_act(elem_t* out, const elem_t* act, const elem_t* w, int M, int N, int K, int64_t lda, int64_t ldo, int activation,
+                hipStream_t st) {
+  return gemm_launch(out, act, w, M, N, K, lda, ldo, 0, activation, st);
 }
 
 // 1 if vk_gemm_swiglu takes these sizes (the caller otherwise runs vk_gemm and vk_swiglu, with the same result).
@@ -1469,7 +1504,7 @@ int vk_gemm_swiglu(elem_t* out, const elem_t* act, const elem_t* w, int M, int I
     return launch_mid<4, 1, true>(out, act, w, M, I, K, lda, ldo, ok4, st);
   }
   const int ntiles = (I + 15) / 16;
-  const int vec_ok = (ldo % 4 == 0) && ((uintptr_t)out % 16 == 0);
+  const int form = (ldo % 4 == 0) && ((uintptr_t)out % 16 == 0);
 #define SWIGLU_STREAMW(W, MT, RC, NW)                                                                       \
   do {                                                                                                     \
     static int resident = 0;                                                                               \
@@ -1482,7 +1517,7 @@ int vk_gemm_swiglu(elem_t* out, const elem_t* act, const elem_t* w, int M, int I
       resident = (cus > 0 ? cus : 256) * (per_cu > 0 ? per_cu : 1);                                        \
     }                                                                                                      \
     gemm_stream_swiglu_kernel<W, MT, RC, NW><<<ntiles < resident ? ntiles : resident, 64 * NW, 0, st>>>(   \
-        out, act, w, M, I, K, lda, ldo, vec_ok);                                                           \
+        out, act, w, M, I, K, lda, ldo, form);                                                           \
   } while (0)
 #define SWIGLU_STREAM(W, MT, RC) SWIGLU_STREAMW(W, MT, RC, SK_WAVES)
   const int nw = M <= 16 ? stream_waves(K / KC) : SK_WAVES;       // as in vk_gemm
@@ -1553,8 +1588,8 @@ int vk_gemm_split_preferred(int M, int rows, int K, int swiglu) {
 // out = act w^T (swiglu 0: w [rows, K], out [M, rows]) or silu(act w_gate^T) * (act w_up^T) (swiglu 1:
 // w = [gate rows; up rows], out [M, rows / 2]), through chunk sums in a workspace: the bits of vk_gemm and
 // vk_gemm_swiglu.  Calls that overlap in time need workspaces of their own.
-int vk_gemm_split(elem_t* out, const elem_t* act, const elem_t* w, int M, int rows, int K, int64_t lda, int64_t ldo,
-                  int swiglu, float* workspace, int64_t workspace_floats, hipStream_t st) {
+static int gemm_split_launch(elem_t* out, const elem_t* act, const elem_t* w, int M, int rows, int K, int64_t lda, int64_t ldo,
+                             int swiglu, int activation, float* workspace, int64_t workspace_floats, hipStream_t st) {
   const int64_t need = vk_gemm_split_floats(M, rows, K, swiglu);
   VK_REQUIRE(need > 0, "gemm_split: sizes M=%d rows=%d K=%d are not supported", M, rows, K);
   VK_REQUIRE(workspace != nullptr && workspace_floats >= need && ((uintptr_t)workspace % 16) == 0,
@@ -1563,12 +1598,12 @@ int vk_gemm_split(elem_t* out, const elem_t* act, const elem_t* w, int M, int ro
   VK_REQUIRE(lda >= K && lda % VK_VEC == 0 && ldo >= out_cols, "gemm_split: bad row strides");
   VK_REQUIRE(((uintptr_t)act % 16) == 0 && ((uintptr_t)w % 16) == 0, "gemm_split: operands must be 16-byte aligned");
 #ifdef VK_BF16
-  const int vec_ok = (ldo % 4 == 0) && ((uintptr_t)out % 16 == 0);
+  const int form = out_form_of(out, ldo, activation);
   const int mt = (M + 15) / 16;
-  if (mt == 1) return launch_split<1>(out, act, w, M, rows, K, lda, ldo, swiglu, workspace, vec_ok, st);
-  if (mt == 2) return launch_split<2>(out, act, w, M, rows, K, lda, ldo, swiglu, workspace, vec_ok, st);
-  if (mt == 3) return launch_split<3>(out, act, w, M, rows, K, lda, ldo, swiglu, workspace, vec_ok, st);
-  return launch_split<4>(out, act, w, M, rows, K, lda, ldo, swiglu, workspace, vec_ok, st);
+  if (mt == 1) return launch_split<1>(out, act, w, M, rows, K, lda, ldo, swiglu, workspace, form, st);
+  if (mt == 2) return launch_split<2>(out, act, w, M, rows, K, lda, ldo, swiglu, workspace, form, st);
+  if (mt == 3) return launch_split<3>(out, act, w, M, rows, K, lda, ldo, swiglu, workspace, form, st);
+  return launch_split<4>(out, act, w, M, rows, K, lda, ldo, swiglu, workspace, form, st);
 #else
   (void)out; (void)st;
   return vk_fail("gemm_split: built for 16-bit elements only");

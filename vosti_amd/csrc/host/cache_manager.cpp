@@ -303,6 +303,12 @@ int CacheManager::state_slot(RequestId id) const {
   return it == requests_.end() ? -1 : it->second.slot;
 }
 
+int32_t CacheManager::token(RequestId id, int position) const {
+  auto it = requests_.find(id);
+  if (it == requests_.end() || position < 0 || position >= (int)it->second.tokens.size()) return -1;
+  return it->second.tokens[position];
+}
+
 int CacheManager::num_logical_pages(RequestId id, int group) const {
   auto it = requests_.find(id);
   if (it == requests_.end() || group < 0 || group >= (int)groups_.size()) return -1;

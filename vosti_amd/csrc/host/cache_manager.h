@@ -76,6 +76,7 @@ class CacheManager {
   int length(RequestId id) const;        // tokens committed
   int pending(RequestId id) const;       // tokens of the step in flight
   int state_slot(RequestId id) const;
+  int32_t token(RequestId id, int position) const;   // the request's token there (committed or of the step in flight), -1 if it has none
   int num_logical_pages(RequestId id, int group) const;   // block-table width this request needs
   // Pages this request could take right now: free ones plus evictable cached ones.
   int available_pages(int group) const;

@@ -61,6 +61,7 @@ int vh_cache_has_request(void* h, uint64_t id) { return CM->has_request(id) ? 1 
 int vh_cache_length(void* h, uint64_t id) { return CM->length(id); }
 int vh_cache_pending(void* h, uint64_t id) { return CM->pending(id); }
 int vh_cache_state_slot(void* h, uint64_t id) { return CM->state_slot(id); }
+int vh_cache_token(void* h, uint64_t id, int position) { return CM->token(id, position); }
 int vh_cache_num_logical_pages(void* h, uint64_t id, int g) { return CM->num_logical_pages(id, g); }
 int vh_cache_available_pages(void* h, int g) { return CM->available_pages(g); }
 int vh_cache_free_pages(void* h, int g) { return CM->free_pages(g); }
@@ -217,6 +218,10 @@ void vh_rotary_linear_frequencies(double theta, int rotary_dim, double factor, f
 float vh_rotary_stretched_frequencies(double theta, int rotary_dim, double factor, double original, double fast, double slow, float* out) {
   return rotary_stretched_frequencies(theta, rotary_dim, factor, original, fast, slow, out);
 }
+void vh_rotary_banded_frequencies(double theta, int rotary_dim, double factor, double original, double low, double high, float* out) {
+  rotary_banded_frequencies(theta, rotary_dim, factor, original, low, high, out);
+}
+int vh_distance_class(int64_t n, int64_t rows, double far) { return distance_class(n, rows, far); }
 int vh_graph_row_bucket(int rows) { return graph_row_bucket(rows); }
 int vh_graph_width_bucket(int pages) { return graph_width_bucket(pages); }
 int vh_max_graphs(void) { return kMaxGraphs; }

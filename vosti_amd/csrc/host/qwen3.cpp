@@ -12,6 +12,7 @@
 #include "kelisun.h"
 #include "pasovik.h"
 #include "povatar.h"
+#include "puvirax.h"
 #include "tezinex.h"
 
 namespace vosti {
@@ -198,6 +199,7 @@ void register_builtin_architectures() {
   register_architecture("Pabavik", "pabavik", pabavik_model_spec);
   register_architecture("Pasovik", "pasovik", pasovik_model_spec);
   register_architecture("Kelisun", "kelisun", kelisun_model_spec);
+  register_architecture("Puvirax", "puvirax", puvirax_model_spec);
 }
 
 }  // namespace vosti

@@ -37,6 +37,28 @@ void rotary_linear_frequencies(double theta, int rotary_dim, double factor, floa
   for (int j = 0; j < rotary_dim / 2; ++j) out[j] = (float)(std::pow(theta, -2.0 * j / rotary_dim) / factor);
 }
 
+void rotary_banded_frequencies(double theta, int rotary_dim, double factor, double original, double low, double high, float* out) {
+  const double pi = 3.14159265358979323846;
+  for (int j = 0; j < rotary_dim / 2; ++j) {
+    const double f = std::pow(theta, -2.0 * j / rotary_dim), wavelength = 2.0 * pi / f;
+    double g = f;
+    if (wavelength > original / low) {
+      g = f / factor;
+    } else if (wavelength >= original / high && high > low) {
+      const double s = (original / wavelength - low) / (high - low);
+      g = (1.0 - s) * f / factor + s * f;
+    }
+    out[j] = (float)g;
+  }
+}
+
+int distance_class(int64_t n, int64_t rows, double far) {
+  const int64_t half = rows / 2;
+  if (n < half) return (int)n;
+  const double place = std::log((double)n / (double)half) / std::log(far / (double)half) * (double)(rows - half);
+  return (int)std::min<double>((double)(rows - 1), (double)half + std::floor(place));
+}
+
 static int bucket(int n) {      // the smallest of 1, 2, 3, 4, 6, 8, 12, 16, ... that is at least n
   for (int b = 1;; b *= 2) {
     if (b >= n) return b;

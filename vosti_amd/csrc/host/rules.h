@@ -3,6 +3,7 @@
 // could differ in a last bit (of a rotation frequency) or in a bucket's border, and with them the logits or
 // the recorded graphs.
 #pragma once
+#include <cstdint>
 
 namespace vosti {
 
@@ -25,6 +26,15 @@ float rotary_stretched_frequencies(double theta, int rotary_dim, double factor, 
 // The frequencies of a rotation whose positions are all stretched alike: out[j] = theta^(-2j / rotary_dim) / factor,
 // computed in 64-bit and rounded once.  factor 1: the plain frequencies.
 void rotary_linear_frequencies(double theta, int rotary_dim, double factor, float* out);
+
+// The frequencies of a rotation that treats bands of wavelengths apart: with f[j] = theta^(-2j / rotary_dim) and its wavelength
+// w = 2 pi / f[j], out[j] = f[j] for w < original / high, f[j] / factor for w > original / low, and between the two
+// (1 - s) f[j] / factor + s f[j] with s = (original / w - low) / (high - low); computed in 64-bit and rounded once.
+void rotary_banded_frequencies(double theta, int rotary_dim, double factor, double original, double low, double high, float* out);
+
+// The class of a distance n >= 0 among `rows`: one each for the distances below rows / 2, then logarithmic ones,
+// min(rows - 1, half + floor(ln(n / half) / ln(far / half) * (rows - half))) with half = rows / 2 (rounded down).
+int distance_class(int64_t n, int64_t rows, double far);
 
 // Recorded decode steps have one of 1, 2, 3, 4, 6, 8, 12, 16, 24, ... rows (a step with fewer is filled up with
 // rows that read one key and store nothing; the reference pads its graphs likewise,

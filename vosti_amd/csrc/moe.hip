@@ -68,9 +68,9 @@ __device__ __forceinline__ void wave_lds_fence() {
   __builtin_amdgcn_wave_barrier();
 }
 
-// The place of the largest of v[0 .. n) over a wave (the lower index wins a tie; values above -2).
+// The place of the largest of v[0 .. n) over a wave (the lower index wins a tie; -inf is never the largest).
 __device__ __forceinline__ int wave_argmax(const float* v, int n, int lane, float& best) {
-  best = -2.f;
+  best = -INFINITY;
   int at = 0x7fffffff;
   for (int i = lane; i < n; i += 64) {
     const float x = v[i];
@@ -89,10 +89,13 @@ __device__ __forceinline__ int wave_argmax(const float* v, int n, int lane, floa
 // score 0: the softmax over all experts, the chosen scores divided by their sum plus weight_eps; score 1: the logistic
 // function of every logit, the chosen scores as they are (the order of the scores is the order of the logits either way);
 // score 2: the softmax over all experts, the chosen scores as they are.  Every weight is multiplied by `scale` at the end.
-// groups > 1 with keep < groups: the experts form that many equal runs of neighbours; a group's score is its largest, and
-// only experts of the `keep` best groups can be chosen.
+// groups > 1 with keep < groups: the experts form that many equal runs of neighbours; a group's score is its largest
+// (group_score 0) or the sum of its two largest (1), and only experts of the `keep` best groups can be chosen.
+// correction (score 1 only; [E] elements or floats, or null): a number an expert that joins its score for the choice, of groups
+// and of experts, and not its weight.  Scores so corrected may be negative.
 __global__ __launch_bounds__(256) void moe_choose_kernel(int32_t* __restrict__ idx, float* __restrict__ wts, const float* __restrict__ logits,
-                                                         int T, int E, int top, float weight_eps, int score_kind, int groups, int keep, float scale) {
+                                                         int T, int E, int top, float weight_eps, int score_kind, int groups, int keep, float scale,
+                                                         int group_score, const void* __restrict__ correction, int correction_is_f32) {
   extern __shared__ float scores[];      // [4][E], then [4][groups]
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int t = blockIdx.x * 4 + wave;
@@ -107,43 +110,47 @@ __global__ __launch_bounds__(256) void moe_choose_kernel(int32_t* __restrict__ i
   float sum = 0.f;
   for (int e = lane; e < E; e += 64) {
     const float p = score_kind == 1 ? 1.f / (1.f + expf(-z[e])) : expf(z[e] - mx);
-    z[e] = p;
+    z[e] = correction != nullptr ? p + load_weight(correction, correction_is_f32, e) : p;
     sum = sum + p;
   }
   sum = score_kind == 1 ? 1.f : wave_sum_xor(sum);
   if (keep < groups) {
-    // A kept group's score is marked with -1; the experts of the others are then marked as if they had been chosen.
+    // A kept group's score is marked with -inf; the experts of the others are then marked as if they had been chosen.
     float* gs = scores + 4 * E + wave * groups;
     const int size = E / groups;
     wave_lds_fence();
     for (int g = lane; g < groups; g += 64) {
-      float m = -1.f;
-      for (int j = 0; j < size; ++j) m = fmaxf(m, z[g * size + j]);
-      gs[g] = fmaxf(m, 0.f);
+      float m = -INFINITY, second = -INFINITY;
+      for (int j = 0; j < size; ++j) {
+        const float v = z[g * size + j];
+        second = fmaxf(second, fminf(m, v));
+        m = fmaxf(m, v);
+      }
+      gs[g] = group_score == 1 && size > 1 ? m + second : m;
     }
     wave_lds_fence();
     for (int k = 0; k < keep; ++k) {
       float best;
       const int g = wave_argmax(gs, groups, lane, best);
-      if (lane == 0) gs[g] = -1.f;
+      if (lane == 0) gs[g] = -INFINITY;
       wave_lds_fence();
     }
     for (int e = lane; e < E; e += 64)
-      if (gs[e / size] >= 0.f) z[e] = -1.f;
+      if (gs[e / size] > -INFINITY) z[e] = -INFINITY;
     wave_lds_fence();
   }
-  // The largest score `top` times; a chosen one is marked with -1 (scores are positive or zero).
+  // The largest score `top` times; a chosen one is marked with -inf.
   float chosen_sum = 0.f;
   float my_w = 0.f;
   int my_e = 0;
   for (int k = 0; k < top; ++k) {
     float best;
     const int best_e = wave_argmax(z, E, lane, best);
-    const float score = best / sum;
+    const float score = correction != nullptr ? 1.f / (1.f + expf(-logits[(int64_t)t * E + best_e])) : best / sum;
     chosen_sum = chosen_sum + score;
     if (lane == k % 64 && k < 64) { my_w = score; my_e = best_e; }
     if (k >= 64 && lane == 0) { idx[(int64_t)t * top + k] = best_e; wts[(int64_t)t * top + k] = score; }
-    if (lane == 0) z[best_e] = -1.f;
+    if (lane == 0) z[best_e] = -INFINITY;
     wave_lds_fence();
   }
   const float denom = score_kind == 0 ? chosen_sum + weight_eps : 1.f;
@@ -385,7 +392,8 @@ int vk_moe_max_tiles(int T, int top, int E, int tile_rows) {
 
 // logits: scratch [T, E] floats.  bias [E] (elements, or floats with bias_is_f32) or null.
 static int route_launch(int32_t* idx, float* wts, float* logits, const elem_t* h, const elem_t* router, const void* bias, int bias_is_f32, int T, int W,
-                        int E, int top, float weight_eps, hipStream_t st, int score_kind = 0, int groups = 1, int keep = 1, float scale = 1.f) {
+                        int E, int top, float weight_eps, hipStream_t st, int score_kind = 0, int groups = 1, int keep = 1, float scale = 1.f, int group_score = 0,
+                        const void* correction = nullptr, int correction_is_f32 = 0) {
   VK_REQUIRE(T >= 0 && W > 0 && W % VK_VEC == 0 && E > 0 && top > 0 && top <= E && E <= 4096,
              "router: bad sizes T=%d W=%d E=%d top=%d (the width in whole 16-byte vectors, at most 4096 experts)", T, W, E, top);
   VK_REQUIRE(((uintptr_t)h % 16) == 0 && ((uintptr_t)router % 16) == 0, "router: operands must be 16-byte aligned");
@@ -400,7 +408,8 @@ static int route_launch(int32_t* idx, float* wts, float* logits, const elem_t* h
   if (vk_check_launch("router (logits)")) return 1;
   const size_t lds = (size_t)4 * (E + (keep < groups ? groups : 0)) * sizeof(float);
   VK_REQUIRE(lds <= 65536, "router: %d experts in %d groups are too many", E, groups);
-  moe_choose_kernel<<<(T + 3) / 4, 256, lds, st>>>(idx, wts, logits, T, E, top, weight_eps, score_kind, groups, keep, scale);
+  moe_choose_kernel<<<(T + 3) / 4, 256, lds, st>>>(idx, wts, logits, T, E, top, weight_eps, score_kind, groups, keep, scale,
+                                                        group_score, correction, correction_is_f32);
   return vk_check_launch("router (choice)");
 }
 
@@ -425,6 +434,15 @@ int vk_moe_route_scored(int32_t* idx, float* wts, float* logits, const elem_t* h
                         int E, int top, float weight_eps, int score_kind, int groups, int keep, float scale, hipStream_t st) {
   VK_REQUIRE(score_kind >= 0 && score_kind <= 2, "router: score kind %d", score_kind);
   return route_launch(idx, wts, logits, h, router, bias, bias_is_f32, T, W, E, top, weight_eps, st, score_kind, groups, keep, scale);
+}
+
+// vk_moe_route_scored with score 1 (logistic scores as they are) and a correction [E] (elements, or floats with
+// correction_is_f32) that joins the scores for the choice of groups and experts and not for the weights; group_score 0: a group
+// is worth its largest corrected score, 1: the sum of its two largest.
+int vk_moe_route_corrected(int32_t* idx, float* wts, float* logits, const elem_t* h, const elem_t* router, const void* correction, int correction_is_f32,
+                           int T, int W, int E, int top, int groups, int keep, int group_score, float scale, hipStream_t st) {
+  VK_REQUIRE(correction != nullptr && (group_score == 0 || group_score == 1), "router: the correction is missing, or group score %d", group_score);
+  return route_launch(idx, wts, logits, h, router, nullptr, 0, T, W, E, top, 0.f, st, 1, groups, keep, scale, group_score, correction, correction_is_f32);
 }
 
 int vk_moe_plan(const int32_t* idx, int32_t* row_pair, int32_t* row_token, int32_t* pair_row, int32_t* tile_expert, int32_t* expert_start, int T,

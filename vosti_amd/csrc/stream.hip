@@ -85,6 +85,23 @@ __global__ __launch_bounds__(STREAM_THREADS) void stream_norm_add_kernel(float* 
   }
 }
 
+// x <- x + y (rows of the stream, in place), out (elements) = norm of the new row: a sublayer's output joins the stream in the
+// launch that reads it for the next one.
+template <typename Y>     // the sublayer's rows: elements, or floats
+__global__ __launch_bounds__(STREAM_THREADS) void stream_add_norm_kernel(elem_t* __restrict__ out, float* __restrict__ x, const Y* __restrict__ y,
+                                                                         const void* __restrict__ w, int w_is_f32, int H, float eps) {
+  __shared__ float red[4];
+  const int64_t base = (int64_t)blockIdx.x * H;
+  float part = 0.f;
+  for (int c = threadIdx.x; c < H; c += STREAM_THREADS) {
+    const float v = x[base + c] + to_f32(y[base + c]);
+    x[base + c] = v;                                      // this thread reads it again below
+    part = part + v * v;
+  }
+  const float rr = rsqrtf(stream_block_sum(part, red) / (float)H + eps);
+  for (int c = threadIdx.x; c < H; c += STREAM_THREADS) out[base + c] = from_f32<elem_t>((x[base + c] * rr) * load_weight(w, w_is_f32, c));
+}
+
 // The same two norms for rows of whole 16-byte vectors that fit a workgroup's registers: thread t owns the vectors t,
 // t + 256, ... (NV of them at most), reads them once, and sums their squares element by element in that order.
 template <bool IN_F32, int NV>
@@ -169,6 +186,52 @@ __global__ __launch_bounds__(STREAM_THREADS) void stream_norm_add_vec_kernel(flo
   }
 }
 
+template <int NV, typename Y>
+__global__ __launch_bounds__(STREAM_THREADS) void stream_add_norm_vec_kernel(elem_t* __restrict__ out, float* __restrict__ x, const Y* __restrict__ y,
+                                                                             const void* __restrict__ w, int w_is_f32, int H, float eps) {
+  __shared__ float red[4];
+  const int64_t base = (int64_t)blockIdx.x * H;
+  const int nvec = H / 4;
+  f32x4 v[NV];
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = threadIdx.x + j * STREAM_THREADS;
+    v[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (c < nvec) {
+      f32x4 u;
+      if constexpr (sizeof(Y) == 4) u = *reinterpret_cast<const f32x4*>(y + base + 4 * c);
+      else u = load_elems4(y + base + 4 * c);
+      v[j] = *reinterpret_cast<const f32x4*>(x + base + 4 * c);
+      v[j].x = v[j].x + u.x;
+      v[j].y = v[j].y + u.y;
+      v[j].z = v[j].z + u.z;
+      v[j].w = v[j].w + u.w;
+    }
+  }
+  float part = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    part = part + v[j].x * v[j].x;
+    part = part + v[j].y * v[j].y;
+    part = part + v[j].z * v[j].z;
+    part = part + v[j].w * v[j].w;
+  }
+  const float rr = rsqrtf(stream_block_sum(part, red) / (float)H + eps);
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = threadIdx.x + j * STREAM_THREADS;
+    if (c < nvec) {
+      *reinterpret_cast<f32x4*>(x + base + 4 * c) = v[j];
+      f32x4 o;
+      o.x = (v[j].x * rr) * load_weight(w, w_is_f32, 4 * c);
+      o.y = (v[j].y * rr) * load_weight(w, w_is_f32, 4 * c + 1);
+      o.z = (v[j].z * rr) * load_weight(w, w_is_f32, 4 * c + 2);
+      o.w = (v[j].w * rr) * load_weight(w, w_is_f32, 4 * c + 3);
+      store_elems4(out + base + 4 * c, o);
+    }
+  }
+}
+
 // out[e] = sum over j < n of coef[j] * states[j * stride + e], added in ascending j from zero.
 __global__ __launch_bounds__(256) void stream_mix_kernel(float* __restrict__ out, const float* __restrict__ states, int64_t stride,
                                                          const void* __restrict__ coef, int coef_is_f32, int n, int64_t numel) {
@@ -215,6 +278,26 @@ __global__ __launch_bounds__(STREAM_THREADS) void embed_scaled_kernel(float* __r
   const elem_t* src = table + (int64_t)ids[blockIdx.x] * H;
   float* dst = out + (int64_t)blockIdx.x * H;
   for (int c = threadIdx.x; c < H; c += blockDim.x) dst[c] = to_f32(src[c]) * scale;
+}
+
+// out[t, :] = table[ids[t], :] + pairs[row, :] as floats, row = (before[t] * mul_before + ids[t] * mul_own) mod buckets, or `buckets`
+// (one row more) where before[t] is negative: a sequence's first token has no predecessor.
+__global__ __launch_bounds__(STREAM_THREADS) void embed_bigram_kernel(float* __restrict__ out, const elem_t* __restrict__ table,
+                                                                      const elem_t* __restrict__ pairs, const int32_t* __restrict__ ids,
+                                                                      const int32_t* __restrict__ before, int H, int64_t mul_before, int64_t mul_own,
+                                                                      int64_t buckets) {
+  const int64_t own = ids[blockIdx.x], prev = before[blockIdx.x];
+  const int64_t row = prev < 0 ? buckets : (prev * mul_before + own * mul_own) % buckets;
+  const elem_t *a = table + own * H, *b = pairs + row * H;
+  float* dst = out + (int64_t)blockIdx.x * H;
+  if (H % 4 == 0) {
+    for (int c = 4 * threadIdx.x; c < H; c += 4 * blockDim.x) {
+      const f32x4 u = load_elems4(a + c), v = load_elems4(b + c);
+      *reinterpret_cast<f32x4*>(dst + c) = f32x4{u.x + v.x, u.y + v.y, u.z + v.z, u.w + v.w};
+    }
+  } else {
+    for (int c = threadIdx.x; c < H; c += blockDim.x) dst[c] = to_f32(a[c]) + to_f32(b[c]);
+  }
 }
 
 // out = base + (a + b) (b may be null: out = base + a), element by element; a and b are floats or elements.
@@ -378,6 +461,40 @@ int vk_stream_norm_add_f32_rounded(float* out, const float* base, const float* y
                                    float mult, elem_t* rounded, hipStream_t st) {
   VK_REQUIRE(rounded != nullptr, "stream norm-add: the rounded rows have no memory");
   return norm_add_launch<float>(out, base, y, w, w_is_f32, rows, H, eps, offset, mult, st, rounded);
+}
+
+extern "C++" {
+template <typename Y>
+static int add_norm_launch(elem_t* out, float* x, const Y* y, const void* w, int w_is_f32, int rows, int H, float eps, hipStream_t st) {
+  VK_REQUIRE(rows >= 0 && H > 0 && eps >= 0.f, "stream add-norm: bad sizes rows=%d H=%d", rows, H);
+  if (rows == 0) return 0;
+  const int nv = (H / 4 + STREAM_THREADS - 1) / STREAM_THREADS;
+  if (H % 4 == 0 && nv <= 8 && (uintptr_t)out % 16 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)y % 16 == 0) {
+#define ADD_NORM_VEC(NV) stream_add_norm_vec_kernel<NV, Y><<<rows, STREAM_THREADS, 0, st>>>(out, x, y, w, w_is_f32, H, eps)
+    if (nv <= 1) ADD_NORM_VEC(1); else if (nv <= 2) ADD_NORM_VEC(2); else if (nv <= 4) ADD_NORM_VEC(4); else ADD_NORM_VEC(8);
+#undef ADD_NORM_VEC
+  } else {
+    stream_add_norm_kernel<Y><<<rows, STREAM_THREADS, 0, st>>>(out, x, y, w, w_is_f32, H, eps);
+  }
+  return vk_check_launch("stream add-norm");
+}
+}  // extern "C++"
+
+// x [rows, H] floats <- x + y (elements, or floats with y_is_f32); out = norm(x) * w as elements.
+int vk_stream_add_norm(elem_t* out, float* x, const void* y, int y_is_f32, const void* w, int w_is_f32, int rows, int H, float eps, hipStream_t st) {
+  if (y_is_f32) return add_norm_launch<float>(out, x, static_cast<const float*>(y), w, w_is_f32, rows, H, eps, st);
+  return add_norm_launch<elem_t>(out, x, static_cast<const elem_t*>(y), w, w_is_f32, rows, H, eps, st);
+}
+
+// pairs [buckets + 1, H].  Ids, and the ids before them (negative: none), must lie below V: the caller checks them on the host.
+int vk_embed_bigram(float* out, const elem_t* table, const elem_t* pairs, const int32_t* ids, const int32_t* before, int T, int H, int V,
+                    int64_t mul_before, int64_t mul_own, int64_t buckets, hipStream_t st) {
+  VK_REQUIRE(T >= 0 && H > 0 && V > 0 && buckets > 0 && mul_before >= 0 && mul_own >= 0 && mul_before < (1ll << 31) && mul_own < (1ll << 31),
+             "bigram embedding: bad sizes T=%d H=%d V=%d buckets=%lld", T, H, V, (long long)buckets);
+  VK_REQUIRE(H % 4 != 0 || ((uintptr_t)out % 16 == 0 && (uintptr_t)table % 16 == 0 && (uintptr_t)pairs % 16 == 0), "bigram embedding: tables must be 16-byte aligned");
+  if (T == 0) return 0;
+  embed_bigram_kernel<<<T, STREAM_THREADS, 0, st>>>(out, table, pairs, ids, before, H, mul_before, mul_own, buckets);
+  return vk_check_launch("bigram embedding");
 }
 
 int vk_stream_mix(float* out, const float* states, int64_t stride, const void* coef, int coef_is_f32, int n, int64_t numel,
