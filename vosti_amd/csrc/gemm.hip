@@ -1605,9 +1605,21 @@ static int gemm_split_launch(elem_t* out, const elem_t* act, const elem_t* w, in
   if (mt == 3) return launch_split<3>(out, act, w, M, rows, K, lda, ldo, swiglu, workspace, form, st);
   return launch_split<4>(out, act, w, M, rows, K, lda, ldo, swiglu, workspace, form, st);
 #else
-  (void)out; (void)st;
+  (void)out; (void)st; (void)activation;
   return vk_fail("gemm_split: built for 16-bit elements only");
 #endif
+}
+
+int vk_gemm_split(elem_t* out, const elem_t* act, const elem_t* w, int M, int rows, int K, int64_t lda, int64_t ldo,
+                  int swiglu, float* workspace, int64_t workspace_floats, hipStream_t st) {
+  return gemm_split_launch(out, act, w, M, rows, K, lda, ldo, swiglu, 0, workspace, workspace_floats, st);
+}
+
+// The plain product of vk_gemm_split with an activation on the outputs.
+int vk_gemm_split_act(elem_t* out, const elem_t* act, const elem_t* w, int M, int rows, int K, int64_t lda, int64_t ldo, int activation,
+                      float* workspace, int64_t workspace_floats, hipStream_t st) {
+  VK_REQUIRE(activation == 0 || activation == 1, "gemm: unknown activation %d", activation);
+  return gemm_split_launch(out, act, w, M, rows, K, lda, ldo, 0, activation, workspace, workspace_floats, st);
 }
 
 }  // extern "C"
