@@ -6,6 +6,7 @@
     python bench.py --workload mixed14b     # Qwen3-14B shape: 32 prompts of 128 to 4,096 tokens, prefill in portions beside decoding
     python bench.py --workload prefix32b    # Qwen3-32B shape: 64 requests at context 8,192 that share a 1,024-token prefix
     python bench.py --workload aligned      # the reference's aligned phases: batch 4, cached contexts 0 to 16K, 256 new tokens / 127 decode steps
+    python bench.py --workload puvirax      # the Puvirax design (three kinds of attention with distance biases, unit norms and blended values, squared-relu layers and experts) at three layer sizes beside Pabavik at equal size
     python bench.py --workload kelisun      # the Kelisun design (windowed attention through a latent, experts chosen by groups, four residual streams, layers that share weights) at three layer sizes beside Pasovik at equal size
     python bench.py --workload pasovik      # the Pasovik design (attention through a latent, linear attention with fixed decays, a second embedding a layer) at three layer sizes beside Pabavik at equal size
     python bench.py --workload pabavik      # the Pabavik design (gated linear attention, windowed attention with an output gate, gated experts beside a shared one) at three layer sizes beside Tezinex at equal size
@@ -90,9 +91,9 @@ def main() -> int:
     ap.add_argument("--no-other-shapes", action="store_true", help="skip the 14B and 32B workloads that the default record holds as points")
     ap.add_argument("--prompt-tokens", type=int, default=PROMPT_TOKENS,
                     help="context length of the decode measurement (the prefill figure is always of 2,048 tokens)")
-    ap.add_argument("--workload", default="decode8b", choices=["decode8b", "mixed14b", "prefix32b", "aligned", "tezinex", "povatar", "pabavik", "pasovik", "kelisun"])
-    ap.add_argument("--sizes", default=",".join(["1k", "2k", "4k"]), help="which layer sizes --workload tezinex / povatar / pabavik / pasovik / kelisun measure (1k, 2k, 4k)")
-    ap.add_argument("--only-design", default="", choices=["", "tezinex", "qwen3", "povatar", "pabavik", "pasovik", "kelisun"], help="--workload tezinex / povatar / pabavik / pasovik / kelisun: measure one of the two designs only")
+    ap.add_argument("--workload", default="decode8b", choices=["decode8b", "mixed14b", "prefix32b", "aligned", "tezinex", "povatar", "pabavik", "pasovik", "kelisun", "puvirax"])
+    ap.add_argument("--sizes", default=",".join(["1k", "2k", "4k"]), help="which layer sizes --workload tezinex / povatar / pabavik / pasovik / kelisun / puvirax measure (1k, 2k, 4k)")
+    ap.add_argument("--only-design", default="", choices=["", "tezinex", "qwen3", "povatar", "pabavik", "pasovik", "kelisun", "puvirax"], help="--workload tezinex / povatar / pabavik / pasovik / kelisun / puvirax: measure one of the two designs only")
     ap.add_argument("--engine", default="native", choices=["native", "python"],
                     help="which engine every figure is measured through: the native one (vosti_amd.engine.NativeEngine) or the "
                          "Python step function over the same kernels, cache manager and scheduler")
@@ -115,7 +116,7 @@ def main() -> int:
     if args.workload == "aligned":
         print(json.dumps(aligned_workload(args)), flush=True)
         return 0
-    if args.workload in ("tezinex", "povatar", "pabavik", "pasovik", "kelisun"):
+    if args.workload in ("tezinex", "povatar", "pabavik", "pasovik", "kelisun", "puvirax"):
         print(json.dumps(tezinex_workload(args)), flush=True)
         return 0
     if args.workload != "decode8b":
@@ -615,12 +616,32 @@ def kelisun_config(width, heads, ff, layers, vocab):
     return {"architecture": "Kelisun", "layers": out, "norm": {"eps": 1e-5}, "streams": 4, "vocab": vocab, "width": width}
 
 
+def puvirax_config(width, heads, kv_heads, ff, layers, vocab):
+    """Attention over a window of 1,024 keys with a bias by distance, attention over all keys with one, rotated attention twice,
+    ... (heads of 128, a 32-row table up to a distance of 128, values blended with the first layer's), in turn a dense
+    squared-relu layer of one and a half times Pabavik's dense size and 32 experts in eight groups of which four are kept, a
+    token using 3 and a shared one, each a quarter of that: two matrices an expert instead of three, so that a token's matrix
+    work is that of a Pabavik layer of these sizes."""
+    common = {"dim": 128, "vdim": 128, "heads": heads, "kv_heads": kv_heads, "v_mix": True}
+    rotated = ("attention", dict(common, scale=128 ** -0.5, rot={"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 2048}}))
+    windowed = ("attention_2", dict(common, scale=128 ** -0.5, bias_max=128, mask={"size": 1024}))
+    unrotated = ("attention_3", dict(common, scale=128 ** -0.5, bias_max=128))
+    dense = {"kind": "dense", "ff": 3 * ff // 2}
+    moe = {"kind": "moe", "expert": {"ff": 3 * ff // 8}, "router": {"experts": 32, "top": 3, "groups": {"count": 8, "keep": 4}}, "shared": {"ff": 3 * ff // 8}}
+    out = []
+    for i in range(layers):
+        kind, mixer = (windowed, unrotated, rotated, rotated)[i % 4]
+        out.append({"type": kind, "mixer": mixer, "mlp": moe if i % 2 else dense})
+    return {"architecture": "Puvirax", "embedding": {"bigram": {"buckets": vocab - 3, "mul_cur": 7, "mul_prev": 31}}, "layers": out, "logit_scale": 0.5,
+            "norm": {"eps": 1e-5}, "vocab": vocab, "width": width}
+
+
 def tezinex_workload(args) -> dict:
     """Prefill of one prompt and decoding at a fixed batch for the Tezinex design at three layer sizes, each beside the
     Qwen3 decoder with the same width, heads, feed-forward, layers and vocabulary (random weights, the native engine).
     --workload povatar: the Povatar design beside Tezinex, its nearest neighbour here, in the same way; --workload pabavik:
     the Pabavik design beside Tezinex; --workload pasovik: the Pasovik design beside Pabavik; --workload kelisun: the Kelisun design
-    beside Pasovik."""
+    beside Pasovik; --workload puvirax: the Puvirax design beside Pabavik."""
     import tempfile
     from vosti_amd.engine import NativeEngine
     from vosti_amd.sampling import SamplingParams
@@ -632,7 +653,8 @@ def tezinex_workload(args) -> dict:
     record = {"metric": "decode_tokens_per_s", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
               "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
               "data": "synthetic: seeded random token prompts, seeded random weights", "sizes": {},
-              "config": {"model": "Kelisun (windowed attention through a latent, 32 experts of which 4, four streams) beside Pasovik at equal size"
+              "config": {"model": "Puvirax (windowed, unrotated and rotated attention; dense squared-relu layers and 32 experts of which 3 and a shared one) beside Pabavik at equal size"
+                         if args.workload == "puvirax" else "Kelisun (windowed attention through a latent, 32 experts of which 4, four streams) beside Pasovik at equal size"
                          if args.workload == "kelisun" else "Pasovik (linear attention, attention, latent attention, attention on the latent before, ...; dense layers and 32 experts of which 4; a second embedding) beside Pabavik at equal size"
                          if args.workload == "pasovik" else "Pabavik (linear attention, attention, shared-key attention, linear attention, ...; 32 experts of which 3 and a shared one) beside Tezinex at equal size"
                          if args.workload == "pabavik" else "Povatar (attention beside a state-space recurrence, 32 experts of which 4) beside Tezinex at equal size"
@@ -685,12 +707,16 @@ def tezinex_workload(args) -> dict:
         first, second = "pasovik", "pabavik"
     if args.workload == "kelisun":
         first, second = "kelisun", "pasovik"
+    if args.workload == "puvirax":
+        first, second = "puvirax", "pabavik"
 
     def config_of(design, width, heads, kv_heads, ff):
         if design == "povatar":
             return povatar_config(width, heads, kv_heads, ff, layers, vocab)
         if design == "pabavik":
             return pabavik_config(width, heads, kv_heads, ff, layers, vocab)
+        if design == "puvirax":
+            return puvirax_config(width, heads, kv_heads, ff, layers, vocab)
         if design == "kelisun":
             return kelisun_config(width, heads, ff, layers, vocab)
         if design == "pasovik":

@@ -96,11 +96,12 @@ __device__ __forceinline__ int wave_argmax(const float* v, int n, int lane, floa
 __global__ __launch_bounds__(256) void moe_choose_kernel(int32_t* __restrict__ idx, float* __restrict__ wts, const float* __restrict__ logits,
                                                          int T, int E, int top, float weight_eps, int score_kind, int groups, int keep, float scale,
                                                          int group_score, const void* __restrict__ correction, int correction_is_f32) {
-  extern __shared__ float scores[];      // [4][E], then [4][groups]
+  extern __shared__ float scores[];      // [4][E], with a correction [4][E] of the scores without it, then [4][groups]
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int t = blockIdx.x * 4 + wave;
   if (t >= T) return;
   float* z = scores + wave * E;
+  float* raw = correction != nullptr ? z + 4 * E : z;
   float mx = -INFINITY;
   for (int e = lane; e < E; e += 64) {
     z[e] = logits[(int64_t)t * E + e];
@@ -110,13 +111,14 @@ __global__ __launch_bounds__(256) void moe_choose_kernel(int32_t* __restrict__ i
   float sum = 0.f;
   for (int e = lane; e < E; e += 64) {
     const float p = score_kind == 1 ? 1.f / (1.f + expf(-z[e])) : expf(z[e] - mx);
-    z[e] = correction != nullptr ? p + load_weight(correction, correction_is_f32, e) : p;
+    raw[e] = p;
+    if (correction != nullptr) z[e] = p + load_weight(correction, correction_is_f32, e);
     sum = sum + p;
   }
   sum = score_kind == 1 ? 1.f : wave_sum_xor(sum);
   if (keep < groups) {
     // A kept group's score is marked with -inf; the experts of the others are then marked as if they had been chosen.
-    float* gs = scores + 4 * E + wave * groups;
+    float* gs = scores + (correction != nullptr ? 8 : 4) * E + wave * groups;
     const int size = E / groups;
     wave_lds_fence();
     for (int g = lane; g < groups; g += 64) {
@@ -139,6 +141,7 @@ __global__ __launch_bounds__(256) void moe_choose_kernel(int32_t* __restrict__ i
       if (gs[e / size] > -INFINITY) z[e] = -INFINITY;
     wave_lds_fence();
   }
+  if (correction != nullptr) wave_lds_fence();
   // The largest score `top` times; a chosen one is marked with -inf.
   float chosen_sum = 0.f;
   float my_w = 0.f;
@@ -146,7 +149,7 @@ __global__ __launch_bounds__(256) void moe_choose_kernel(int32_t* __restrict__ i
   for (int k = 0; k < top; ++k) {
     float best;
     const int best_e = wave_argmax(z, E, lane, best);
-    const float score = correction != nullptr ? 1.f / (1.f + expf(-logits[(int64_t)t * E + best_e])) : best / sum;
+    const float score = correction != nullptr ? raw[best_e] : best / sum;
     chosen_sum = chosen_sum + score;
     if (lane == k % 64 && k < 64) { my_w = score; my_e = best_e; }
     if (k >= 64 && lane == 0) { idx[(int64_t)t * top + k] = best_e; wts[(int64_t)t * top + k] = score; }
@@ -406,7 +409,7 @@ static int route_launch(int32_t* idx, float* wts, float* logits, const elem_t* h
   const int grid_x = groups_of_tokens > 8 ? (groups_of_tokens + 7) / 8 * 8 : groups_of_tokens;
   moe_logits_kernel<<<dim3(grid_x, E), 256, 0, st>>>(logits, h, router, T, W, E, bias, bias_is_f32);
   if (vk_check_launch("router (logits)")) return 1;
-  const size_t lds = (size_t)4 * (E + (keep < groups ? groups : 0)) * sizeof(float);
+  const size_t lds = (size_t)4 * ((correction != nullptr ? 2 : 1) * E + (keep < groups ? groups : 0)) * sizeof(float);
   VK_REQUIRE(lds <= 65536, "router: %d experts in %d groups are too many", E, groups);
   moe_choose_kernel<<<(T + 3) / 4, 256, lds, st>>>(idx, wts, logits, T, E, top, weight_eps, score_kind, groups, keep, scale,
                                                         group_score, correction, correction_is_f32);
