@@ -632,7 +632,7 @@ def puvirax_config(width, heads, kv_heads, ff, layers, vocab):
     for i in range(layers):
         kind, mixer = (windowed, unrotated, rotated, rotated)[i % 4]
         out.append({"type": kind, "mixer": mixer, "mlp": moe if i % 2 else dense})
-    return {"architecture": "Puvirax", "embedding": {"bigram": {"buckets": vocab - 3, "mul_cur": 7, "mul_prev": 31}}, "layers": out, "logit_scale": 0.5,
+    return {"architecture": "Puvirax", "embedding": {"bigram": {"buckets": vocab - 3, "mul_cur": 29, "mul_prev": 13}}, "layers": out, "logit_scale": 0.25,
             "norm": {"eps": 1e-5}, "vocab": vocab, "width": width}
 
 

@@ -79,7 +79,7 @@ WIDE = config([
     layer(unrotated(8, 4, 48, 32, far=48), moe(6, 2, 48, groups=(3, 1), shared=64)),
     layer(rotated(2, 2, 256, 64, dims=256, scale=0.02, mix=True)),
     layer(windowed(2, 1, 200, 128, window=64, far=20), moe(16, 5, 64, groups=(4, 2))),
-], width=104, vocab=130, buckets=509, mul_prev=1, mul_cur=0, logit_scale=3.0, eps=1e-6)
+], width=104, vocab=130, buckets=487, mul_prev=1, mul_cur=0, logit_scale=3.0, eps=1e-6)
 CONFIGS = {"MIXED": MIXED, "WIDE": WIDE}
 
 

@@ -119,7 +119,7 @@ def test_the_banded_frequencies_are_the_plain_ones():
 
 def test_the_distance_classes_are_the_plain_ones():
     from vosti_amd.cache.host import distance_class
-    for rows, far in ((16, 120), (32, 128), (11, 300), (6, 25), (2, 20), (3, 9.5), (7, 4)):
+    for rows, far in ((16, 150), (32, 128), (11, 300), (6, 25), (2, 20), (3, 9.5), (7, 4)):
         assert [distance_class(n, rows, far) for n in range(700)] == [plain.distance_class(n, rows, far) for n in range(700)]
 
 
@@ -152,8 +152,8 @@ def test_norms_against_torch():
 
 
 def test_rows_of_pairs():
-    b = {"buckets": 10, "mul_prev": 3, "mul_cur": 7}
-    assert plain.bigram_rows(b, [4, 9, 9, 0]) == [10, (3 * 4 + 7 * 9) % 10, (3 * 9 + 7 * 9) % 10, (3 * 9) % 10]
+    b = {"buckets": 10, "mul_prev": 3, "mul_cur": 17}
+    assert plain.bigram_rows(b, [4, 9, 9, 0]) == [10, (3 * 4 + 17 * 9) % 10, (3 * 9 + 17 * 9) % 10, (3 * 9) % 10]
 
 
 def test_bands_written_out():

@@ -553,6 +553,22 @@ def test_greedy_generation_through_the_scheduler(models, graphs):
             assert list(got) == plain.generate_greedy(cfg, w, prompt, 12)
 
 
+def test_a_shared_prefix_is_found_and_its_last_token_remembered(tmp_path):
+    """Without windows pages are kept for later requests: a prompt that starts like an earlier one goes on behind the matched
+    pages, where the embedding needs the token before."""
+    from vosti_amd.engine import create_engine
+    from vosti_amd.sampling.params import SamplingParams
+    cfg = config([layer(rotated(2, 1, 16, 16, dims=8), dense(24)), layer(unrotated(4, 2, 8, 8, far=30))], width=32, vocab=60)
+    w = random_weights(cfg, 12)
+    folder = write_model(tmp_path / "prefix", cfg, w)
+    eng = create_engine(folder, dtype="float32", num_pages=24, page_size=16, max_num_seqs=2, enable_prefix_cache=True)
+    shared = tokens_for(cfg, 48, 90)
+    for tail in (5, 9, 16):
+        prompt = shared + tokens_for(cfg, tail, 91 + tail)
+        assert list(eng.generate([prompt], SamplingParams(max_tokens=6, ignore_eos=True))[0]) == plain.generate_greedy(cfg, w, prompt, 6)
+    assert eng.stats()["prefix_hits"] >= 6
+
+
 def test_the_command_line_generates_the_plain_tokens(models):
     """The engine's program, started as a user starts it with --family puvirax: greedy tokens of the plain implementation."""
     import subprocess
